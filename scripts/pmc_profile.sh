@@ -13,13 +13,15 @@ mkdir -p "$OUT"
 
 run_pmc () {
   local name="$1"; shift
-  rocprofv3 --pmc "$@" -d "$OUT/$name" --output-format csv -- \
-    python /root/repo/scripts/gpu_attn_bench.py > "$OUT/$name.log" 2>&1 || true
+  timeout -s KILL 120 rocprofv3 --pmc "$@" -d "$OUT/$name" \
+    --output-format csv -- \
+    python /root/repo/scripts/gpu_attn_bench.py > "$OUT/$name.log" 2>&1
 }
 
-# one counter set per run (hardware counter slots are limited)
-run_pmc mfma   SQ_VALU_MFMA_BUSY_CYCLES SQ_BUSY_CYCLES
-run_pmc lds    SQ_LDS_BANK_CONFLICT SQ_LDS_IDX_ACTIVE
-run_pmc mem    TCC_REQ_sum TCC_HIT_sum TCC_MISS_sum
-run_pmc waves  SQ_WAVES SQ_WAIT_ANY_CYCLES
+# one counter set per run (hardware counter slots are limited); the first
+# run that fails ends the script
+run_pmc mfma   SQ_VALU_MFMA_BUSY_CYCLES SQ_BUSY_CYCLES &&
+run_pmc lds    SQ_LDS_BANK_CONFLICT SQ_LDS_IDX_ACTIVE &&
+run_pmc mem    TCC_REQ_sum TCC_HIT_sum TCC_MISS_sum &&
+run_pmc waves  SQ_WAVES SQ_WAIT_ANY_CYCLES &&
 echo "PMC outputs in $OUT — keep only the small CSV summaries for profiles/"

@@ -10,45 +10,53 @@ from __future__ import annotations
 
 import importlib.util
 import os
-from typing import Optional
+from typing import Dict
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
-_SO = os.path.join(_HERE, "_quoracle_ops.so")
 
-_ext = None
-_load_error: Optional[str] = None
+_loaded: Dict[str, object] = {}
+_load_errors: Dict[str, str] = {}
 
 
-def _load():
-    global _ext, _load_error
-    if _ext is not None:
-        return _ext
-    if not os.path.exists(_SO):
-        _load_error = f"native extension not built: {_SO} missing " \
-                      "(run quoracle_amd/ops/build.py)"
+def _load(name: str):
+    if name in _loaded:
+        return _loaded[name]
+    path = os.path.join(_HERE, name + ".so")
+    if not os.path.exists(path):
+        _load_errors[name] = f"native extension not built: {path} missing " \
+                             "(run quoracle_amd/ops/build.py)"
         return None
     try:
-        spec = importlib.util.spec_from_file_location("_quoracle_ops", _SO)
+        spec = importlib.util.spec_from_file_location(name, path)
         mod = importlib.util.module_from_spec(spec)
         spec.loader.exec_module(mod)
-        _ext = mod
     except Exception as exc:  # noqa: BLE001
-        _load_error = f"native extension failed to load: {exc}"
+        _load_errors[name] = f"native extension failed to load: {exc}"
         return None
-    return _ext
+    _loaded[name] = mod
+    return mod
+
+
+def _require(name: str):
+    mod = _load(name)
+    if mod is None:
+        raise RuntimeError(
+            f"quoracle_amd HIP extension unavailable: {_load_errors[name]}")
+    return mod
 
 
 def available() -> bool:
-    return _load() is not None
+    return _load("_quoracle_ops") is not None
 
 
 def ext():
     """The native module; raises loudly when missing (no silent fallback)."""
-    mod = _load()
-    if mod is None:
-        raise RuntimeError(
-            f"quoracle_amd HIP extension unavailable: {_load_error}")
-    return mod
+    return _require("_quoracle_ops")
+
+
+def hybrid_ext():
+    """The native module of the hybrid models; raises when missing."""
+    return _require("_quoracle_hybrid")
 
 
 # -- thin wrappers -----------------------------------------------------------

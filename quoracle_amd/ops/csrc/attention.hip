@@ -11,7 +11,7 @@
 // panel is BLOCK_SIZE*D*2 bytes contiguous, so both phases read contiguous
 // rows.
 
-#include "common.h"
+#include "attention_core.h"
 
 #define MAX_GQ 8      // query heads per KV head (llama3-8b: 4)
 #define CHUNK 128     // KV tokens processed per software chunk
@@ -441,33 +441,9 @@ paged_attn_decode_reduce_kernel(bf16 *__restrict__ out,
                                 const float *__restrict__ part_l,
                                 const float *__restrict__ part_acc,
                                 int Hq, int D, int NS) {
-  const int b = blockIdx.x;
-  const int h = blockIdx.y;
-  const int tid = threadIdx.x;
-  const long base = ((long)b * Hq + h) * NS;
-
-  float M = -INFINITY;
-  for (int i = tid; i < NS; i += blockDim.x)
-    M = fmaxf(M, part_m[base + i]);
-  __shared__ float scratch[8];
-  M = block_max(M, scratch);
-
-  float L = 0.f;
-  for (int i = tid; i < NS; i += blockDim.x) {
-    float mi = part_m[base + i];
-    L += (mi == -INFINITY) ? 0.f : part_l[base + i] * __expf(mi - M);
-  }
-  L = block_sum(L, scratch);
-
-  if (tid < D) {
-    float o = 0.f;
-    for (int i = 0; i < NS; ++i) {
-      float mi = part_m[base + i];
-      if (mi == -INFINITY) continue;
-      o = fmaf(part_acc[(base + i) * D + tid], __expf(mi - M), o);
-    }
-    out[((long)b * Hq + h) * D + tid] = f2bf(L > 0.f ? o / L : 0.f);
-  }
+  const long row = (long)blockIdx.x * Hq + blockIdx.y;
+  attn_core::combine_splits(out + row * D, part_m, part_l, part_acc, row * NS,
+                            1, D, NS);
 }
 
 // ---------------------------------------------------------------------------
@@ -624,31 +600,10 @@ paged_attn_prefill_reduce_kernel(bf16 *__restrict__ out,
   const int tile = blockIdx.x;
   const int h = blockIdx.y;
   const int qi = blockIdx.z;
-  const int tid = threadIdx.x;
-  const int q0 = tile_q0[tile];
   if (qi >= tile_qn[tile]) return;
-  __shared__ float scratch[8];
-
-  const long base0 = (((long)tile * Hq + h) * NS) * QT + qi;
-  float M = -INFINITY;
-  for (int i = tid; i < NS; i += blockDim.x)
-    M = fmaxf(M, part_m[base0 + (long)i * QT]);
-  M = block_max(M, scratch);
-  float L = 0.f;
-  for (int i = tid; i < NS; i += blockDim.x) {
-    float mi = part_m[base0 + (long)i * QT];
-    L += (mi == -INFINITY) ? 0.f : part_l[base0 + (long)i * QT] * __expf(mi - M);
-  }
-  L = block_sum(L, scratch);
-  if (tid < D) {
-    float o = 0.f;
-    for (int i = 0; i < NS; ++i) {
-      float mi = part_m[base0 + (long)i * QT];
-      if (mi == -INFINITY) continue;
-      o = fmaf(part_acc[(base0 + (long)i * QT) * D + tid], __expf(mi - M), o);
-    }
-    out[((long)(q0 + qi) * Hq + h) * D + tid] = f2bf(L > 0.f ? o / L : 0.f);
-  }
+  const long row = (long)(tile_q0[tile] + qi) * Hq + h;
+  attn_core::combine_splits(out + row * D, part_m, part_l, part_acc,
+                            (((long)tile * Hq + h) * NS) * QT + qi, QT, D, NS);
 }
 
 // ---------------------------------------------------------------------------

@@ -1,0 +1,283 @@
+// Elementwise, norm and gate kernels of the hybrid (recurrent + attention)
+// models.  T is the activation type (bf16 or float); the residual stream, all
+// norms, gates of a recurrence and position angles are float32.
+//
+// VEC = 4 kernels need every row start to be a multiple of 4 elements.
+
+#include "hybrid_common.h"
+
+// ---------------------------------------------------------------------------
+// x[t] = embed[tokens[t]] (+ table[positions[t]]); h = T(x).
+// Grid: (T); block 256.
+// ---------------------------------------------------------------------------
+template <typename T, int VEC>
+__global__ void __launch_bounds__(256)
+embed_positions_kernel(float *__restrict__ x, T *__restrict__ h,
+                       const T *__restrict__ embed,
+                       const T *__restrict__ table,
+                       const int *__restrict__ tokens,
+                       const int *__restrict__ positions, int n) {
+  const long t = blockIdx.x;
+  const T *e = embed + (long)tokens[t] * n;
+  const T *p = table ? table + (long)positions[t] * n : nullptr;
+  for (int i = threadIdx.x * VEC; i < n; i += 256 * VEC) {
+    float a[VEC], b[VEC];
+    hyb::load_v<VEC>(e + i, a);
+    if (p) {
+      hyb::load_v<VEC>(p + i, b);
+#pragma unroll
+      for (int k = 0; k < VEC; ++k) a[k] += b[k];
+    }
+    hyb::store_v<VEC>(x + t * n + i, a);
+    hyb::store_v<VEC>(h + t * n + i, a);
+  }
+}
+
+// ---------------------------------------------------------------------------
+// Norm after the sum: x <- rms(alpha*x + sa*a (+ sb*b)) * w in place;
+// h = T(x).  Grid: (T); block 256.
+// ---------------------------------------------------------------------------
+template <typename T, int VEC>
+__global__ void __launch_bounds__(256)
+post_norm_kernel(float *__restrict__ x, T *__restrict__ h,
+                 const T *__restrict__ a, float sa, const T *__restrict__ b,
+                 float sb, float alpha, const float *__restrict__ w, int n,
+                 float eps) {
+  __shared__ float scratch[4];
+  const long row = (long)blockIdx.x * n;
+  float ssq = 0.f;
+  for (int i = threadIdx.x * VEC; i < n; i += 256 * VEC) {
+    float xv[VEC], av[VEC], bv[VEC];
+    hyb::load_v<VEC>(x + row + i, xv);
+    hyb::load_v<VEC>(a + row + i, av);
+#pragma unroll
+    for (int k = 0; k < VEC; ++k) xv[k] = alpha * xv[k] + sa * av[k];
+    if (b) {
+      hyb::load_v<VEC>(b + row + i, bv);
+#pragma unroll
+      for (int k = 0; k < VEC; ++k) xv[k] += sb * bv[k];
+    }
+#pragma unroll
+    for (int k = 0; k < VEC; ++k) ssq += xv[k] * xv[k];
+    hyb::store_v<VEC>(x + row + i, xv);
+  }
+  const float inv = 1.f / sqrtf(block_sum(ssq, scratch) / (float)n + eps);
+  // each thread re-reads only what it wrote itself
+  for (int i = threadIdx.x * VEC; i < n; i += 256 * VEC) {
+    float xv[VEC], wv[VEC];
+    hyb::load_v<VEC>(x + row + i, xv);
+    hyb::load_v<VEC>(w + i, wv);
+#pragma unroll
+    for (int k = 0; k < VEC; ++k) xv[k] = xv[k] * inv * wv[k];
+    hyb::store_v<VEC>(x + row + i, xv);
+    hyb::store_v<VEC>(h + row + i, xv);
+  }
+}
+
+// ---------------------------------------------------------------------------
+// out[r] = T(rms(x[rows[r]]) * w): the final norm of the rows that need
+// logits.  Grid: (R); block 256.
+// ---------------------------------------------------------------------------
+template <typename T, int VEC>
+__global__ void __launch_bounds__(256)
+norm_rows_kernel(T *__restrict__ out, const float *__restrict__ x,
+                 const long *__restrict__ rows, const float *__restrict__ w,
+                 int n, float eps) {
+  __shared__ float scratch[4];
+  const float *src = x + rows[blockIdx.x] * (long)n;
+  T *dst = out + (long)blockIdx.x * n;
+  float ssq = 0.f;
+  for (int i = threadIdx.x * VEC; i < n; i += 256 * VEC) {
+    float v[VEC];
+    hyb::load_v<VEC>(src + i, v);
+#pragma unroll
+    for (int k = 0; k < VEC; ++k) ssq += v[k] * v[k];
+  }
+  const float inv = 1.f / sqrtf(block_sum(ssq, scratch) / (float)n + eps);
+  for (int i = threadIdx.x * VEC; i < n; i += 256 * VEC) {
+    float v[VEC], wv[VEC];
+    hyb::load_v<VEC>(src + i, v);
+    hyb::load_v<VEC>(w + i, wv);
+#pragma unroll
+    for (int k = 0; k < VEC; ++k) v[k] = v[k] * inv * wv[k];
+    hyb::store_v<VEC>(dst + i, v);
+  }
+}
+
+// ---------------------------------------------------------------------------
+// out = silu(gu[:, :n]) * gu[:, n:].  Grid: (T, ceil(n / (256*VEC))).
+// ---------------------------------------------------------------------------
+template <typename T, int VEC>
+__global__ void __launch_bounds__(256)
+glu_kernel(T *__restrict__ out, const T *__restrict__ gu, int n) {
+  const long t = blockIdx.x;
+  const int i = (blockIdx.y * 256 + threadIdx.x) * VEC;
+  if (i >= n) return;
+  float g[VEC], u[VEC];
+  hyb::load_v<VEC>(gu + t * 2 * n + i, g);
+  hyb::load_v<VEC>(gu + t * 2 * n + n + i, u);
+#pragma unroll
+  for (int k = 0; k < VEC; ++k) g[k] = g[k] * hyb::sigmoid_f(g[k]) * u[k];
+  hyb::store_v<VEC>(out + t * n + i, g);
+}
+
+// ---------------------------------------------------------------------------
+// Norm each group of `n` values of o[t] (a head, or all heads together),
+// times w[n], times act(gate): out[t, g*n + i].  The gate is read in place
+// from the fused projection row.  Grid: (T, groups); block = multiple of 64.
+// ---------------------------------------------------------------------------
+template <typename T, int VEC>
+__global__ void __launch_bounds__(256)
+gated_norm_kernel(T *__restrict__ out, const T *__restrict__ o,
+                  const T *__restrict__ proj, long stride, int g_off,
+                  const float *__restrict__ w, int n, int act, float eps) {
+  __shared__ float scratch[4];
+  const long t = blockIdx.x;
+  const long base = (t * gridDim.y + blockIdx.y) * (long)n;
+  const T *gate = proj + t * stride + g_off + (long)blockIdx.y * n;
+  const int step = blockDim.x * VEC;
+  float ssq = 0.f;
+  for (int i = threadIdx.x * VEC; i < n; i += step) {
+    float v[VEC];
+    hyb::load_v<VEC>(o + base + i, v);
+#pragma unroll
+    for (int k = 0; k < VEC; ++k) ssq += v[k] * v[k];
+  }
+  const float inv = 1.f / sqrtf(block_sum(ssq, scratch) / (float)n + eps);
+  for (int i = threadIdx.x * VEC; i < n; i += step) {
+    float v[VEC], gv[VEC], wv[VEC];
+    hyb::load_v<VEC>(o + base + i, v);
+    hyb::load_v<VEC>(gate + i, gv);
+    hyb::load_v<VEC>(w + i, wv);
+#pragma unroll
+    for (int k = 0; k < VEC; ++k)
+      v[k] = v[k] * inv * wv[k] * hyb::activate(gv[k], act);
+    hyb::store_v<VEC>(out + base + i, v);
+  }
+}
+
+// ---------------------------------------------------------------------------
+// Attention input of one token, fused: RMS norm over the whole query and over
+// the whole key projection, rotation of the interleaved pairs (2i, 2i+1) of
+// the first 2*n_pairs dimensions of each head by pos * freq[i] (cos and sin
+// times `mag`), queries out, rotated keys and the raw projected keys (the
+// values) into the paged cache.
+// Grid: (T); block 256; dynamic LDS 2*n_pairs floats.
+// ---------------------------------------------------------------------------
+template <typename T>
+__global__ void __launch_bounds__(256)
+qk_norm_rope_store_kernel(
+    T *__restrict__ q_out, T *__restrict__ kcache, T *__restrict__ vcache,
+    const T *__restrict__ proj, long stride, int q_off, int k_off,
+    const float *__restrict__ qw, const float *__restrict__ kw,
+    const int *__restrict__ positions, const int *__restrict__ slots,
+    const double *__restrict__ freq, int n_pairs, float mag, float eps, int H,
+    int G, int D, int BS) {
+  extern __shared__ float rot_s[];
+  __shared__ float scratch[4];
+  float *cos_s = rot_s, *sin_s = rot_s + n_pairs;
+  const long t = blockIdx.x;
+  const int tid = threadIdx.x;
+  const T *qp = proj + t * stride + q_off;
+  const T *kp = proj + t * stride + k_off;
+  const int nq = H * D, nk = G * D;
+  const double pos = (double)positions[t];
+  for (int i = tid; i < n_pairs; i += 256) {
+    // whole turns taken off before the angle becomes a float
+    double turns = pos * freq[i] * 0.15915494309189535;
+    turns -= rint(turns);
+    float s, c;
+    sincosf((float)(turns * 6.283185307179586), &s, &c);
+    cos_s[i] = c * mag;
+    sin_s[i] = s * mag;
+  }
+  float sq = 0.f, sk = 0.f;
+  for (int i = tid; i < nq; i += 256) {
+    const float v = hyb::to_f(qp[i]);
+    sq += v * v;
+  }
+  for (int i = tid; i < nk; i += 256) {
+    const float v = hyb::to_f(kp[i]);
+    sk += v * v;
+  }
+  const float qi = 1.f / sqrtf(block_sum(sq, scratch) / (float)nq + eps);
+  const float ki = 1.f / sqrtf(block_sum(sk, scratch) / (float)nk + eps);
+
+  const int slot = slots[t];
+  const long blk = slot / BS;
+  const int off = slot % BS;
+  const int hp = (D + 1) / 2;                    // pairs per head
+  for (int p = tid; p < (H + G) * hp; p += 256) {
+    const int head = p / hp, pr = p % hp;
+    const bool is_q = head < H;
+    const int i0 = (is_q ? head : head - H) * D + 2 * pr;
+    const bool two = 2 * pr + 1 < D;
+    const T *src = is_q ? qp : kp;
+    const float *w = is_q ? qw : kw;
+    const float inv = is_q ? qi : ki;
+    const float r0 = hyb::to_f(src[i0]);
+    const float r1 = two ? hyb::to_f(src[i0 + 1]) : 0.f;
+    float u = r0 * inv * w[i0];
+    float v = two ? r1 * inv * w[i0 + 1] : 0.f;
+    if (pr < n_pairs) {
+      const float c = cos_s[pr], s = sin_s[pr];
+      const float a = u * c - v * s;
+      v = v * c + u * s;
+      u = a;
+    }
+    if (is_q) {
+      T *dst = q_out + t * nq + i0;
+      hyb::put(dst, u);
+      if (two) hyb::put(dst + 1, v);
+    } else if (slot >= 0) {
+      const long at =
+          ((blk * G + (head - H)) * (long)BS + off) * D + 2 * pr;
+      hyb::put(kcache + at, u);
+      hyb::put(vcache + at, r0);
+      if (two) {
+        hyb::put(kcache + at + 1, v);
+        hyb::put(vcache + at + 1, r1);
+      }
+    }
+  }
+}
+
+// ---------------------------------------------------------------------------
+// Log of a low-rank sigmoid decay per key channel, summed along runs of
+// consecutive rows:
+//   z = A2 a1[t] + b,  ld[t] = log(sigmoid(z)) / tau,
+//   out[t] = ld[t] + out[t-1] inside a run (the first row of a run: ld[t]).
+// run_row0 null: every row is a run of its own (out = ld).
+// Grid: (runs, ceil(C/256)); block 256, one channel per thread.
+// ---------------------------------------------------------------------------
+template <typename T>
+__global__ void __launch_bounds__(256)
+log_decay_kernel(float *__restrict__ out, const T *__restrict__ proj,
+                 long stride, int a_off, int rank, const T *__restrict__ a2,
+                 const float *__restrict__ bias, float inv_tau, int C,
+                 const int *__restrict__ run_row0,
+                 const int *__restrict__ run_len) {
+  const int c = blockIdx.y * 256 + threadIdx.x;
+  if (c >= C) return;
+  const long row0 = run_row0 ? run_row0[blockIdx.x] : (int)blockIdx.x;
+  const int len = run_row0 ? run_len[blockIdx.x] : 1;
+  const T *wr = a2 + (long)c * rank;
+  float w[16];
+#pragma unroll
+  for (int r = 0; r < 16; ++r) w[r] = r < rank ? hyb::to_f(wr[r]) : 0.f;
+  const float b = bias[c];
+  float sum = 0.f;
+  for (int t = 0; t < len; ++t) {
+    const T *a = proj + (row0 + t) * stride + a_off;
+    float z = 0.f;
+#pragma unroll
+    for (int r = 0; r < 16; ++r)
+      if (r < rank) z = fmaf(w[r], hyb::to_f(a[r]), z);
+    for (int r = 16; r < rank; ++r)
+      z = fmaf(hyb::to_f(wr[r]), hyb::to_f(a[r]), z);
+    z += b;
+    const float ls = fminf(z, 0.f) - log1pf(expf(-fabsf(z)));
+    sum += ls * inv_tau;
+    out[(row0 + t) * (long)C + c] = sum;
+  }
+}

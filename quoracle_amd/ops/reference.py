@@ -143,3 +143,116 @@ def gather_rows(out: torch.Tensor, src: torch.Tensor,
                 rows: torch.Tensor) -> torch.Tensor:
     out.copy_(src[rows.long()])
     return out
+
+
+# -- hybrid models: recurrent mixers and chunk-local attention ---------------
+
+def _rms(x: torch.Tensor, w: torch.Tensor, eps: float) -> torch.Tensor:
+    return x * torch.rsqrt(x.square().mean(-1, keepdim=True) + eps) * w.float()
+
+
+def _act(x: torch.Tensor, act: int) -> torch.Tensor:
+    """0 none, 1 silu, 2 sigmoid (the kernels' selectors)."""
+    if act == 1:
+        return torch.nn.functional.silu(x)
+    return torch.sigmoid(x) if act == 2 else x
+
+
+def embed_positions(x, h, embed, table, tokens, positions) -> None:
+    v = embed[tokens.long()].float()
+    if table is not None:
+        v = v + table[positions.long()].float()
+    x.copy_(v)
+    h.copy_(v)
+
+
+def post_norm(x, h, a, sa, b, sb, alpha, w, eps) -> None:
+    y = alpha * x + sa * a.float()
+    if b is not None:
+        y = y + sb * b.float()
+    x.copy_(_rms(y, w, eps))
+    h.copy_(x)
+
+
+def norm_rows(out, x, rows, w, eps) -> None:
+    out.copy_(_rms(x[rows], w, eps))
+
+
+def gated_norm(out, o, proj, g_off, w, groups, act, eps) -> None:
+    T, n = o.shape[0], w.shape[0]
+    y = _rms(o.float().view(T, groups, n), w, eps).view(T, groups * n)
+    gate = proj[:, g_off:g_off + groups * n].float()
+    out.copy_((y * _act(gate, act)).view_as(out))
+
+
+def rope_interleaved(x: torch.Tensor, pos: torch.Tensor, freq: torch.Tensor,
+                     mag: float) -> torch.Tensor:
+    """Rotate the pairs (2i, 2i+1), i < len(freq), of x [T, H, D]."""
+    n = freq.shape[0]
+    ang = pos.double()[:, None] * freq.double()[None, :]
+    cos = (ang.cos().float() * mag)[:, None, :]
+    sin = (ang.sin().float() * mag)[:, None, :]
+    pairs = x[..., :2 * n].unflatten(-1, (n, 2))
+    u, v = pairs[..., 0], pairs[..., 1]
+    turned = torch.stack([u * cos - v * sin, v * cos + u * sin], dim=-1)
+    return torch.cat([turned.flatten(-2), x[..., 2 * n:]], dim=-1)
+
+
+def qk_norm_rope_store(q_out, kcache, vcache, proj, q_off, k_off, qw, kw,
+                       positions, slots, freq, mag, eps) -> None:
+    T, H, D = q_out.shape
+    G = kcache.shape[1]
+    raw = proj[:, k_off:k_off + G * D].float()
+    q = _rms(proj[:, q_off:q_off + H * D].float(), qw, eps).view(T, H, D)
+    k = _rms(raw, kw, eps).view(T, G, D)
+    q_out.copy_(rope_interleaved(q, positions, freq, mag))
+    k = rope_interleaved(k, positions, freq, mag).to(kcache.dtype)
+    kv_append(kcache, vcache, k, raw.view(T, G, D).to(vcache.dtype), slots)
+
+
+def local_attention(out, q, kcache, vcache, block_tables, row_seq, positions,
+                    scale, chunk, sink) -> None:
+    gq = q.shape[1] // kcache.shape[1]
+    for seq in row_seq.unique().tolist():
+        rows = (row_seq == seq).nonzero(as_tuple=True)[0]
+        pos = positions[rows].long()
+        length = int(pos.max()) + 1
+        k = _gather_kv(kcache, block_tables[seq], length).float()
+        v = _gather_kv(vcache, block_tables[seq], length).float()
+        k, v = k.repeat_interleave(gq, 1), v.repeat_interleave(gq, 1)
+        s = torch.einsum("qhd,khd->hqk", q[rows].float(), k) * scale
+        key = torch.arange(length)
+        ok = key[None, :] <= pos[:, None]
+        if chunk > 0:
+            ok &= (key // chunk)[None, :] == (pos // chunk)[:, None]
+        s = s.masked_fill(~ok[None], float("-inf"))
+        if sink:
+            s = torch.cat([s, torch.zeros_like(s[..., :1])], dim=-1)
+        p = torch.softmax(s, dim=-1)[..., :length]
+        out[rows] = torch.einsum("hqk,khd->qhd", p, v).to(out.dtype)
+
+
+def log_decay(out, proj, a_off, a2, bias, tau) -> None:
+    a = proj[:, a_off:a_off + a2.shape[1]].float()
+    z = a @ a2.float().T + bias
+    out.copy_(torch.nn.functional.logsigmoid(z) / tau)
+
+
+def linear_attention(o, proj, q_off, k_off, v_off, act, qscale, decay,
+                     channel, state, slots, row_seq, positions) -> None:
+    H, V, D = state.shape[1:]
+    T = proj.shape[0]
+    q = _act(proj[:, q_off:q_off + H * D].float(), act).view(T, H, D)
+    k = _act(proj[:, k_off:k_off + H * D].float(), act).view(T, H, D)
+    v = _act(proj[:, v_off:v_off + H * V].float(), act).view(T, H, V)
+    a = decay.exp().view(T, H, D) if channel \
+        else decay[None, :, None].expand(T, H, D)
+    y = torch.empty(T, H, V)
+    for t in range(T):          # rows of a sequence come in order
+        slot = int(slots[int(row_seq[t])])
+        if int(positions[t]) == 0:
+            state[slot].zero_()
+        S = state[slot]
+        S.mul_(a[t][:, None, :]).add_(v[t][:, :, None] * k[t][:, None, :])
+        y[t] = (S @ q[t][:, :, None]).squeeze(-1) * qscale
+    o.copy_(y.view_as(o))

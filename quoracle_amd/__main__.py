@@ -6,6 +6,10 @@
       and the web monitor on http://HOST:PORT.
   python -m quoracle_amd show-prompts [scenario]
       Render verbatim LLM prompts (reference: mix quoracle.show_llm_prompts).
+  python -m quoracle_amd generate --model KEY --prompt TEXT
+      One reply of one model (a preset, or a checkpoint folder).
+  python -m quoracle_amd trace-run --model DIR --out DIR --max-tokens N
+      Replay given token ids and write logits (same as bin/trace_run).
 """
 
 from __future__ import annotations
@@ -63,12 +67,39 @@ def cmd_serve(args) -> None:
     uvicorn.run(app, host=args.host, port=args.port, log_level="warning")
 
 
+def cmd_generate(args) -> None:
+    import torch
+
+    from .engine.api import GenerateRequest
+    from .engine.engine import LocalEngine
+    device = torch.device(args.device) if args.device else None
+    engine = LocalEngine([args.model], device=device, embed_model_key=None,
+                         kv_gb_per_model=args.kv_gb,
+                         dtype=getattr(torch, args.dtype))
+    result = engine.generate_sync(GenerateRequest(
+        model_key=args.model,
+        messages=[{"role": "user", "content": args.prompt}],
+        temperature=args.temperature, max_tokens=args.max_tokens,
+        seed=args.seed))
+    if not result.ok:
+        raise SystemExit(f"generate failed: {result.error}")
+    print(result.text)
+    print(f"[generate] {result.input_tokens} in, {result.output_tokens} out, "
+          f"{result.latency_ms:.0f} ms", file=sys.stderr)
+
+
 def main() -> None:
+    # everything after "trace-run" is that program's own
+    if sys.argv[1:2] == ["trace-run"]:
+        from .tools.trace_run import main as trace_run
+        raise SystemExit(trace_run(sys.argv[2:]))
     p = argparse.ArgumentParser(prog="quoracle_amd")
     sub = p.add_subparsers(dest="cmd", required=True)
 
     s = sub.add_parser("serve", help="engine + runtime + web monitor")
-    s.add_argument("--models", default="llama3-8b#0,llama3-8b#1,llama3-8b#2")
+    s.add_argument("--models", default="llama3-8b#0,llama3-8b#1,llama3-8b#2",
+                   help="comma-separated model keys: a preset or a "
+                        "checkpoint folder, each optionally #INSTANCE")
     s.add_argument("--db", default="quoracle.db")
     s.add_argument("--host", default="127.0.0.1")
     s.add_argument("--port", type=int, default=8800)
@@ -79,6 +110,23 @@ def main() -> None:
     s.add_argument("--fake", action="store_true",
                    help="FakeEngine backend (no GPU; orchestrator demo)")
     s.set_defaults(fn=cmd_serve)
+
+    g = sub.add_parser("generate", help="one reply of one model")
+    g.add_argument("--model", required=True,
+                   help="preset or checkpoint folder")
+    g.add_argument("--prompt", required=True)
+    g.add_argument("--max-tokens", type=int, default=64)
+    g.add_argument("--temperature", type=float, default=0.0,
+                   help="0: greedy")
+    g.add_argument("--seed", type=int, default=None)
+    g.add_argument("--dtype", choices=["bfloat16", "float32"],
+                   default="bfloat16",
+                   help="float32: hybrid models only")
+    g.add_argument("--kv-gb", type=float, default=1.0)
+    g.add_argument("--device", default=None)
+    g.set_defaults(fn=cmd_generate)
+
+    sub.add_parser("trace-run", help="replay given token ids, write logits")
 
     sp = sub.add_parser("show-prompts", help="render verbatim LLM prompts")
     sp.add_argument("scenario", nargs="?", default="all")

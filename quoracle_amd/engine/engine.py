@@ -21,6 +21,7 @@ reference: lib/quoracle/models/model_query.ex):
 from __future__ import annotations
 
 import asyncio
+import contextlib
 import os
 import queue
 import sys
@@ -32,17 +33,20 @@ from typing import Dict, List, Optional, Sequence, Tuple
 import numpy as np
 import torch
 
-from ..models import LlamaModel, get_config
+from ..models import LlamaModel, build_model, get_config
 from .api import Engine, GenerateRequest, GenerateResult
 from .graphs import DecodeGraphs
-from .kv_cache import BlockManager, OutOfBlocks, Session, SessionCache
+from .kv_cache import (BlockManager, OutOfBlocks, Session, SessionCache,
+                       StateSlots)
 from .sampler import FORCED, ActionGrammar, Sampler, SamplingParams
-from .tokenizer import ByteTokenizer, EOS
-from ..models.llama import ForwardBatch, KVCache
+from .tokenizer import VOCAB_FLOOR, ByteTokenizer, EOS
+from ..models.llama import ForwardBatch
+from ..ops.hybrid import ATTN_TILE, LIN_CHUNK
 
 BLOCK_SIZE = 16
 PREFILL_CHUNK = 2048         # max prefill tokens per model per engine step
 QT = 16                      # prefill tile height (must match attention.hip)
+STATE_SLOTS = 64             # sequences with a recurrent state held at once
 
 # $/1M tokens (input, output) per preset — budget plumbing needs real-ish
 # numbers (reference records per-call costs: lib/quoracle/costs/recorder.ex)
@@ -72,15 +76,29 @@ class _Seq:
         return self.prompt + self.emitted
 
 
+@dataclass
+class BatchEntry:
+    """One sequence's part of a step: its next tokens, and the places among
+    them whose logits are wanted."""
+    session: Session
+    tokens: List[int]
+    want: Sequence[int] = ()
+    seq: Optional[_Seq] = None
+    error: Optional[str] = None          # set when the cache has no room
+
+
 class _HostedModel:
     def __init__(self, key: str, device: torch.device, kv_blocks: int,
-                 tp=None):
+                 tp=None, dtype: torch.dtype = torch.bfloat16,
+                 state_slots: int = STATE_SLOTS):
         self.key = key
         self.cfg = get_config(key)
-        self.model = LlamaModel(key, device, tp=tp)
-        self.kv: KVCache = self.model.new_kv_cache(kv_blocks, BLOCK_SIZE)
+        self.model = build_model(key, device, dtype=dtype, tp=tp)
+        self.kv = self.model.new_kv_cache(kv_blocks, BLOCK_SIZE,
+                                          state_slots=state_slots)
+        self.state_slots = state_slots
         self.mgr = BlockManager(kv_blocks, BLOCK_SIZE)
-        self.sessions = SessionCache(self.mgr)
+        self.sessions = self._new_sessions()
         self.active: List[_Seq] = []
         self.sampler = Sampler(self.cfg.vocab_size, device)
         # each hosted model launches on its own HIP stream so pool members
@@ -97,10 +115,26 @@ class _HostedModel:
             # stack; TP decode stays eager until proven
             self.graphs.enabled = False
 
+    def _new_sessions(self) -> SessionCache:
+        return SessionCache(self.mgr, StateSlots(self.state_slots)
+                            if self.cfg.needs_state else None)
+
     def stream_ctx(self):
-        import contextlib
         return (torch.cuda.stream(self.stream) if self.stream is not None
                 else contextlib.nullcontext())
+
+
+def _to_device(arrays: Dict[str, Sequence[int]],
+               device: torch.device) -> Dict[str, torch.Tensor]:
+    """int32 arrays as views of one buffer: a single host-to-device copy."""
+    host = {k: np.asarray(v, dtype=np.int32) for k, v in arrays.items()}
+    flat = torch.from_numpy(
+        np.concatenate([a.ravel() for a in host.values()])).to(device)
+    out, at = {}, 0
+    for k, a in host.items():
+        out[k] = flat[at:at + a.size].view(a.shape)
+        at += a.size
+    return out
 
 
 class LocalEngine(Engine):
@@ -110,7 +144,8 @@ class LocalEngine(Engine):
                  embed_model_key: Optional[str] = "embed-small",
                  kv_blocks_override: Optional[int] = None,
                  prefill_chunk: int = PREFILL_CHUNK,
-                 tp=None):
+                 tp=None, dtype: torch.dtype = torch.bfloat16,
+                 state_slots: int = STATE_SLOTS):
         self.device = device or torch.device(
             "cuda:0" if torch.cuda.is_available() else "cpu")
         self.tokenizer = ByteTokenizer()
@@ -121,12 +156,15 @@ class LocalEngine(Engine):
             if kv_blocks_override is not None:
                 blocks = kv_blocks_override
             else:
-                per_block = cfg.kv_bytes_per_token() * BLOCK_SIZE
+                per_block = max(1, cfg.kv_bytes_per_token(dtype.itemsize)
+                                * BLOCK_SIZE)
                 blocks = max(8, int(kv_gb_per_model * (1 << 30) / per_block))
                 # small models would otherwise allocate millions of blocks
                 # for the same byte budget; 2M tokens of KV is plenty
                 blocks = min(blocks, (2 << 20) // BLOCK_SIZE)
-            self.models[key] = _HostedModel(key, self.device, blocks, tp=tp)
+            self.models[key] = _HostedModel(
+                key, self.device, blocks, tp=tp, dtype=dtype,
+                state_slots=state_slots)
         self.embed_model: Optional[LlamaModel] = None
         if embed_model_key:
             self.embed_model = LlamaModel(embed_model_key, self.device)
@@ -268,6 +306,10 @@ class LocalEngine(Engine):
         if hm is None:
             return GenerateResult(model_key=request.model_key,
                                   error=f"model_not_hosted:{request.model_key}")
+        if hm.cfg.vocab_size < VOCAB_FLOOR:
+            return GenerateResult(
+                model_key=request.model_key,
+                error=f"vocabulary_too_small:{hm.cfg.vocab_size}")
         prompt = self.tokenizer.render_messages(request.messages)
         if len(prompt) > hm.cfg.max_context:
             return GenerateResult(model_key=request.model_key,
@@ -354,6 +396,11 @@ class LocalEngine(Engine):
             seq.result = GenerateResult(
                 model_key=hm.key, error=f"engine_error:{exc}")
         self._finish(hm, crashed)
+        # the failed step may have recorded tokens whose K/V or recurrent
+        # state was never written
+        for seq in crashed:
+            if seq.session is not None:
+                hm.sessions.drop(seq.session.session_id)
         # Watchdog: repeated failures mean corrupted
         # device state — rebuild the model's KV world.  Conversation
         # history lives in the orchestrator, so sessions re-prefill
@@ -380,10 +427,9 @@ class LocalEngine(Engine):
         self._finish(hm, crashed)
         blocks = hm.mgr.num_blocks
         bs = hm.kv.block_size
-        for t in hm.kv.k + hm.kv.v:
-            t.zero_()
+        hm.kv.clear()
         hm.mgr = BlockManager(blocks, bs)
-        hm.sessions = SessionCache(hm.mgr)
+        hm.sessions = hm._new_sessions()
         scratch = hm.mgr.alloc(1)[0]
         hm.graphs.scratch_block = scratch
         hm.crash_count = 0
@@ -424,11 +470,12 @@ class LocalEngine(Engine):
                 self.stats["requests_done"] += 1
 
     def _launch_model(self, hm: _HostedModel):
-        dev = self.device
-        decode: List[_Seq] = []
-        prefill: List[Tuple[_Seq, int]] = []       # (seq, n_new_tokens)
+        """Schedule one step of a model's sequences and run it as one batch.
+        Returns what _sample_model takes, or None when there is nothing."""
+        entries: List[BatchEntry] = []
         early_done: List[_Seq] = []
         budget = self.prefill_chunk
+        active_ids = [s.session.session_id for s in hm.active]
         for seq in hm.active:
             self._expand_forced(hm, seq)
             if seq.finished:
@@ -436,142 +483,171 @@ class LocalEngine(Engine):
                 continue
             cached = len(seq.session.token_ids)
             remaining = len(seq.known) - cached
-            if remaining <= 0:
-                remaining = 1      # shouldn't happen; treat as decode resample
-            if remaining == 1:
-                decode.append(seq)
-            elif budget > 0:
-                n = min(remaining, budget)
+            n = 1 if remaining <= 1 else min(remaining, budget)
+            if n <= 0:
+                continue
+            if not hm.sessions.place(seq.session, active_ids):
+                continue       # every state slot is held: wait for one
+            if n > 1 or remaining > 1:
                 budget -= n
-                prefill.append((seq, n))
+            entries.append(BatchEntry(
+                seq.session, seq.known[cached:cached + n],
+                want=(n - 1,) if n == remaining else (), seq=seq))
 
         if early_done:
             self._finish(hm, early_done)
-        if not decode and not prefill:
+        if not entries:
             return None
+        rows, logits, on_default = self.run_batch(hm, entries, active_ids)
+        failed = []
+        for e in entries:
+            if e.error is not None:
+                e.seq.result = GenerateResult(model_key=hm.key, error=e.error)
+                failed.append(e.seq)
+        if rows is None:
+            self._finish(hm, failed)
+            return None
+        return ([e.seq for e, _ in rows], logits, failed, on_default)
 
-        tokens: List[int] = []
-        positions: List[int] = []
+    def run_batch(self, hm: _HostedModel, entries: Sequence[BatchEntry],
+                  active_ids: Sequence[str]):
+        """Run the entries as ONE mixed batch over the model's cache: single
+        tokens as decode rows, longer runs as prefill rows.
+
+        Returns (rows, logits, on_default_stream): rows lists (entry, place)
+        of each logits row; rows is None when no entry found room (their
+        `error` is set), logits None when none are wanted."""
+        for e in entries:
+            end = len(e.session.token_ids) + len(e.tokens)
+            if not e.tokens or end > hm.cfg.max_context:
+                raise ValueError(
+                    f"{len(e.tokens)} tokens up to position {end} of "
+                    f"{hm.cfg.max_context}")
+            if min(e.tokens) < 0 or max(e.tokens) >= hm.cfg.vocab_size:
+                raise ValueError(f"token outside 0..{hm.cfg.vocab_size - 1}")
+            if any(not 0 <= w < len(e.tokens) for w in e.want):
+                raise ValueError("logits wanted outside the entry's tokens")
+
+        starts: List[int] = []
         slots: List[int] = []
-        bt_rows: List[List[int]] = []
-        ctx_lens: List[int] = []
-        failed: List[_Seq] = []
-        active_ids = [s.session.session_id for s in hm.active]
-
-        def _extend(seq: _Seq, toks: List[int]) -> Optional[List[int]]:
+        placed: List[BatchEntry] = []
+        for e in ([e for e in entries if len(e.tokens) == 1]
+                  + [e for e in entries if len(e.tokens) > 1]):
+            start = len(e.session.token_ids)
             try:
-                return hm.sessions.extend(seq.session, toks, active=active_ids)
+                slots.extend(hm.sessions.extend(e.session, e.tokens,
+                                                active=active_ids))
             except OutOfBlocks as exc:
-                seq.result = GenerateResult(model_key=hm.key,
-                                            error=f"kv_exhausted:{exc}")
-                failed.append(seq)
-                return None
-
-        for seq in decode:
-            cached = len(seq.session.token_ids)
-            tok = seq.known[cached]
-            s = _extend(seq, [tok])
-            if s is None:
+                e.error = f"kv_exhausted:{exc}"
                 continue
-            tokens.append(tok)
-            positions.append(cached)
-            slots.extend(s)
-            bt_rows.append(list(seq.session.blocks))
-            ctx_lens.append(cached + 1)
-        n_decode = len(ctx_lens)
+            starts.append(start)
+            placed.append(e)
+        if not placed:
+            return None, None, False
+        n_decode = sum(1 for e in placed if len(e.tokens) == 1)
 
         # pure-decode steps replay the hipGraph-captured step when possible.
         # Replay + its input copies run on the DEFAULT stream: hipGraph
         # replay launched from a side stream deadlocks on ROCm 7.2 (observed
         # on MI355X; graph kernels never complete), so graph steps serialize
         # across models while eager prefill keeps per-model streams.
-        if n_decode and not prefill:
-            sample_seqs = [s for s in decode if s not in failed]
+        if n_decode == len(placed):
             if hm.stream is not None:
                 # order after this model's eager (prefill) stream, and make
                 # that stream wait for the replay before later prefills
                 torch.cuda.current_stream(self.device).wait_stream(hm.stream)
             logits = hm.graphs.run(
-                tokens, positions, slots, bt_rows, ctx_lens,
+                [e.tokens[0] for e in placed], starts, slots,
+                [e.session.blocks for e in placed], [s + 1 for s in starts],
                 # the full block tuple participates in the staging key:
                 # after eviction + re-prefill a session can reuse the same
                 # length and tail block with different middle blocks
-                bt_keys=[(s.session.session_id,
-                          hash(tuple(s.session.blocks)))
-                         for s in sample_seqs])
-            if logits is not None and hm.stream is not None:
-                hm.stream.wait_stream(torch.cuda.current_stream(self.device))
+                bt_keys=[(e.session.session_id,
+                          hash(tuple(e.session.blocks))) for e in placed],
+                state_slots=[e.session.state_slot for e in placed])
             if logits is not None:
+                if hm.stream is not None:
+                    hm.stream.wait_stream(
+                        torch.cuda.current_stream(self.device))
                 st = self.stats
                 st["engine_steps"] += 1
                 st["graph_steps"] = st.get("graph_steps", 0) + 1
                 st["forward_tokens"] += n_decode
                 st["decode_tokens"] += n_decode
-                return (sample_seqs, logits, failed, True)
+                keep = [i for i, e in enumerate(placed) if len(e.want)]
+                if not keep:
+                    return [], None, True
+                if len(keep) < len(placed):
+                    logits = logits[keep]
+                return [(placed[i], 0) for i in keep], logits, True
+        return self._run_eager(hm, placed, starts, slots, n_decode)
 
-        tile_q0: List[int] = []
-        tile_qn: List[int] = []
-        tile_seq: List[int] = []
-        tile_pos0: List[int] = []
-        t32_q0: List[int] = []
-        t32_qn: List[int] = []
-        t32_seq: List[int] = []
-        t32_pos0: List[int] = []
-        # decode rows sample at their own row index
-        sample_rows: List[int] = list(range(n_decode))
-        sample_seqs: List[_Seq] = [s for s in decode if s not in failed]
-
-        row = n_decode
-        max_kv = 0
-        # 128-row tiles match the default T12 prefill kernel (352 TF,
-        # validated r2); QUORACLE_MFMA64/QUORACLE_MFMA32 fall back
-        if os.environ.get("QUORACLE_MFMA32"):
+    def _run_eager(self, hm: _HostedModel, placed: List[BatchEntry],
+                   starts: List[int], slots: List[int], n_decode: int):
+        dev = self.device
+        tokens: List[int] = []
+        positions: List[int] = []
+        rows: List[Tuple[BatchEntry, int]] = []
+        sample_rows: List[int] = []
+        # 128-row tiles match the default T12 prefill kernel (352 TF);
+        # QUORACLE_MFMA64/QUORACLE_MFMA32 fall back (Llama family)
+        if hm.cfg.is_hybrid:
+            big_step = ATTN_TILE
+        elif os.environ.get("QUORACLE_MFMA32"):
             big_step = 32
         elif os.environ.get("QUORACLE_MFMA64"):
             big_step = 64
         else:
             big_step = 128
-        for seq, n in prefill:
-            cached = len(seq.session.token_ids)
-            chunk = seq.known[cached:cached + n]
-            s = _extend(seq, chunk)
-            if s is None:
+        tiles: Dict[str, List[int]] = {
+            f"{t}_{f}": [] for t in ("tile", "tile32")
+            for f in ("q0", "qn", "seq", "pos0")}
+        row_seq: List[int] = []
+        seg: Dict[str, List[int]] = {"row0": [], "len": [], "chunk0": [0]}
+        chunk: Dict[str, List[int]] = {"row0": [], "len": []}
+        max_kv = 0
+        for i, (e, start) in enumerate(zip(placed, starts)):
+            row, n = len(tokens), len(e.tokens)
+            tokens.extend(e.tokens)
+            positions.extend(range(start, start + n))
+            for w in e.want:
+                rows.append((e, w))
+                sample_rows.append(row + w)
+            row_seq.extend([i] * n)
+            if i < n_decode:
                 continue
-            bt_rows.append(list(seq.session.blocks))
-            seq_row = len(bt_rows) - 1
-            tokens.extend(chunk)
-            positions.extend(range(cached, cached + n))
-            slots.extend(s)
-            for off in range(0, n, QT):
-                tile_q0.append(row + off)
-                tile_qn.append(min(QT, n - off))
-                tile_seq.append(seq_row)
-                tile_pos0.append(cached + off)
-            for off in range(0, n, big_step):
-                t32_q0.append(row + off)
-                t32_qn.append(min(big_step, n - off))
-                t32_seq.append(seq_row)
-                t32_pos0.append(cached + off)
-            if cached + n == len(seq.known):
-                sample_rows.append(row + n - 1)
-                sample_seqs.append(seq)
-            max_kv = max(max_kv, cached + n)
-            row += n
+            max_kv = max(max_kv, start + n)
+            for name, step in (("tile", QT), ("tile32", big_step)):
+                if name == "tile" and hm.cfg.is_hybrid:
+                    continue
+                for off in range(0, n, step):
+                    tiles[name + "_q0"].append(row + off)
+                    tiles[name + "_qn"].append(min(step, n - off))
+                    tiles[name + "_seq"].append(i)
+                    tiles[name + "_pos0"].append(start + off)
+            seg["row0"].append(row)
+            seg["len"].append(n)
+            for off in range(0, n, LIN_CHUNK):
+                chunk["row0"].append(row + off)
+                chunk["len"].append(min(LIN_CHUNK, n - off))
+            seg["chunk0"].append(len(chunk["row0"]))
 
-        if not tokens:
-            self._finish(hm, failed)
-            return None
-
-        maxb = max(len(r) for r in bt_rows)
+        maxb = max(len(e.session.blocks) for e in placed)
         # numpy staging: per-row torch.tensor() creation measured ~20us
         # each on the eager step path
-        bt_np = np.zeros((len(bt_rows), maxb), dtype=np.int32)
-        for i, r in enumerate(bt_rows):
-            bt_np[i, :len(r)] = r
-        bt = torch.from_numpy(bt_np)
-
-        def t32(x):
-            return torch.tensor(x, dtype=torch.int32, device=dev)
+        bt_np = np.zeros((len(placed), maxb), dtype=np.int32)
+        for i, e in enumerate(placed):
+            bt_np[i, :len(e.session.blocks)] = e.session.blocks
+        arrays = {"tokens": tokens, "positions": positions, "slots": slots,
+                  "block_tables": bt_np, **tiles}
+        if n_decode:
+            arrays["ctx_lens"] = [s + 1 for s in starts[:n_decode]]
+        if hm.cfg.is_hybrid:
+            arrays.update(
+                row_seq=row_seq, seg_row0=seg["row0"], seg_len=seg["len"],
+                seg_chunk0=seg["chunk0"], chunk_row0=chunk["row0"],
+                chunk_len=chunk["len"],
+                state_slots=[e.session.state_slot for e in placed])
 
         t_fwd = time.monotonic()
         # rocprof/omnitrace attribution: roctx ranges around each eager
@@ -579,25 +655,17 @@ class LocalEngine(Engine):
         if self._roctx:
             torch.cuda.nvtx.range_push(
                 f"fwd:{hm.key}:T{len(tokens)}:d{n_decode}")
-        # batch tensors are H2D copies: build them on the model's stream so
-        # the forward (same stream) is ordered after them without a sync
+        # batch tensors are one H2D copy: made on the model's stream so the
+        # forward (same stream) is ordered after it without a sync
         with hm.stream_ctx():
             batch = ForwardBatch(
-                tokens=t32(tokens), positions=t32(positions), slots=t32(slots),
-                block_tables=bt.to(dev, non_blocking=False),
-                n_decode=n_decode,
-                ctx_lens=t32(ctx_lens) if n_decode else None,
-                max_ctx=max(ctx_lens) if ctx_lens else 0,
-                max_kv=max_kv,
-                tile_q0=t32(tile_q0), tile_qn=t32(tile_qn),
-                tile_seq=t32(tile_seq), tile_pos0=t32(tile_pos0),
-                tile32_q0=t32(t32_q0), tile32_qn=t32(t32_qn),
-                tile32_seq=t32(t32_seq), tile32_pos0=t32(t32_pos0))
+                n_decode=n_decode, max_ctx=max(starts[:n_decode], default=-1)
+                + 1, max_kv=max_kv, **_to_device(arrays, dev))
             hidden = hm.model.forward(batch, hm.kv)
             logits = None
             if sample_rows:
-                rows = torch.tensor(sample_rows, dtype=torch.long, device=dev)
-                logits = hm.model.compute_logits(hidden, rows)
+                at = torch.tensor(sample_rows, dtype=torch.long, device=dev)
+                logits = hm.model.compute_logits(hidden, at)
         if self._roctx:
             torch.cuda.nvtx.range_pop()
         st = self.stats
@@ -610,11 +678,38 @@ class LocalEngine(Engine):
                   f"T={len(tokens)} dec={n_decode} active={len(hm.active)} "
                   f"launch_ms={(time.monotonic() - t_fwd) * 1e3:.1f}",
                   file=sys.stderr, flush=True)
-        return (sample_seqs, logits, failed, False)
+        return rows, logits, False
+
+    # -- direct stepping -----------------------------------------------------
+
+    def step_entries(self, model_key: str,
+                     entries: Sequence[Tuple[str, Sequence[int],
+                                             Sequence[int]]],
+                     live: Sequence[str] = ()) -> Optional[torch.Tensor]:
+        """Feed given tokens instead of sampled ones: each entry is (session
+        id, next tokens, places wanted), all of them one batch of the same
+        step that generation runs.  Sessions named here or in `live` are not
+        evicted.  Returns the wanted logits in the order of the entries and
+        of their places, [wanted, vocab] float32 on the CPU."""
+        hm = self.models[model_key]
+        batch = [BatchEntry(hm.sessions.get_or_create(sid), list(tokens),
+                            want=tuple(want)) for sid, tokens, want in entries]
+        keep = set(live) | {e.session.session_id for e in batch}
+        with self._gpu_lock:
+            rows, logits, on_default = self.run_batch(hm, batch, list(keep))
+            for e in batch:
+                if e.error is not None:
+                    raise OutOfBlocks(e.error)
+            if not rows:
+                return None
+            with (contextlib.nullcontext() if on_default
+                  else hm.stream_ctx()):
+                out = logits.cpu()
+        at = {(id(e), w): i for i, (e, w) in enumerate(rows)}
+        return out[[at[id(e), w] for e in batch for w in e.want]]
 
     def _sample_model(self, hm: _HostedModel, sample_seqs, logits,
                       failed, on_default_stream=False) -> None:
-        import contextlib
         done: List[_Seq] = list(failed)
         if logits is not None:
             with (contextlib.nullcontext() if on_default_stream

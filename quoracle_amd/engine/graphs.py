@@ -66,6 +66,12 @@ class DecodeGraphs:
                                        dtype=torch.int32, device=dev),
             "ctx_lens": torch.ones(bucket, dtype=torch.int32, device=dev),
         }
+        hybrid = self.kv.state_slots > 0
+        if hybrid:
+            # padding rows sit at position 0 of the scratch state slot
+            bufs["state_slots"] = torch.full(
+                (bucket,), self.kv.state_slots, dtype=torch.int32, device=dev)
+        row_seq = torch.arange(bucket, dtype=torch.int32, device=dev)
         rows = torch.arange(bucket, dtype=torch.long, device=dev)
         scope = __import__("os").environ.get("QUORACLE_GRAPH_SCOPE", "full")
 
@@ -74,7 +80,8 @@ class DecodeGraphs:
                 tokens=bufs["tokens"], positions=bufs["positions"],
                 slots=bufs["slots"], block_tables=bufs["block_tables"],
                 n_decode=bucket, ctx_lens=bufs["ctx_lens"],
-                max_ctx=1 << 30)     # force the split decode path (NS fixed)
+                max_ctx=1 << 30,     # force the split decode path (NS fixed)
+                row_seq=row_seq, state_slots=bufs.get("state_slots"))
             hidden = self.model.forward(batch, self.kv)
             if scope == "noheads":
                 return hidden
@@ -115,8 +122,13 @@ class DecodeGraphs:
             "block_tables": torch.full((bucket, self.maxb), self.scratch_block,
                                        dtype=torch.int32, pin_memory=pin),
         }
+        if hybrid:
+            host["state_slots"] = torch.full(
+                (bucket,), self.kv.state_slots, dtype=torch.int32,
+                pin_memory=pin)
         entry = {"graph": graph, "bufs": bufs, "logits": logits,
-                 "rows": rows, "scope": scope, "host": host,
+                 "rows": rows, "row_seq": row_seq, "scope": scope,
+                 "host": host,
                  "bt_keys": [None] * bucket}
         self.graphs[bucket] = entry
         return entry
@@ -138,7 +150,8 @@ class DecodeGraphs:
 
     def run(self, tokens: List[int], positions: List[int], slots: List[int],
             bt_rows: List[List[int]], ctx_lens: List[int],
-            bt_keys: Optional[List] = None):
+            bt_keys: Optional[List] = None,
+            state_slots: Optional[List[int]] = None):
         """Returns logits[:B] or None if graphs are unavailable.
 
         bt_keys: optional per-row identity (session_id, n_blocks) — rows
@@ -162,6 +175,10 @@ class DecodeGraphs:
                 return None
         bufs, host = entry["bufs"], entry["host"]
         pad_slot = self.scratch_block * self.kv.block_size
+        # the staging buffers are still being read until the last step's
+        # copies have run (a step whose logits nobody reads does not sync)
+        if entry.get("copied") is not None:
+            entry["copied"].synchronize()
         # pinned staging: fill rows 0..B-1 (pad rows persist from capture),
         # then one async H2D per buffer
         host["tokens"][:B] = torch.tensor(tokens, dtype=torch.int32)
@@ -172,6 +189,12 @@ class DecodeGraphs:
         host["slots"][B:] = pad_slot
         host["ctx_lens"][:B] = torch.tensor(ctx_lens, dtype=torch.int32)
         host["ctx_lens"][B:] = 1
+        names = ["tokens", "positions", "slots", "ctx_lens"]
+        if "state_slots" in bufs:
+            host["state_slots"][:B] = torch.tensor(state_slots,
+                                                   dtype=torch.int32)
+            host["state_slots"][B:] = self.kv.state_slots
+            names.append("state_slots")
         bt_host = host["block_tables"]
         keys = entry["bt_keys"]
         bt_dirty = False
@@ -189,10 +212,14 @@ class DecodeGraphs:
                 bt_host[i] = self.scratch_block
                 keys[i] = None
                 bt_dirty = True
-        for name in ("tokens", "positions", "slots", "ctx_lens"):
+        for name in names:
             bufs[name].copy_(host[name], non_blocking=True)
         if bt_dirty or bt_keys is None:
             bufs["block_tables"].copy_(bt_host, non_blocking=True)
+        if bufs["tokens"].is_cuda:
+            if entry.get("copied") is None:
+                entry["copied"] = torch.cuda.Event()
+            entry["copied"].record()
         entry["graph"].replay()
         if entry["scope"] == "noheads":
             return self.model.compute_logits(entry["logits"],

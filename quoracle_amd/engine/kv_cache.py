@@ -10,6 +10,10 @@ physical analogue is a paged KV cache sized for 288 GB HBM3E per GPU:
     calls: on the next call the engine diffs the new prompt against the
     cached token prefix and only prefills the tail (the MI355X replacement
     for the reference's provider prompt cache, consensus_handler.ex:126-152).
+  * StateSlots — models with a recurrent state keep one state per sequence
+    beside the pages; a session holds one slot of that pool.  A state cannot
+    be cut back to an earlier token, so such a session is reused only when
+    the new prompt continues ALL of its tokens, and starts over otherwise.
 """
 
 from __future__ import annotations
@@ -44,12 +48,37 @@ class BlockManager:
         return (n_tokens + self.block_size - 1) // self.block_size
 
 
+class OutOfSlots(OutOfBlocks):
+    pass
+
+
+class StateSlots:
+    """Free list of recurrent-state slots."""
+
+    def __init__(self, num_slots: int):
+        self.num_slots = num_slots
+        self._free: List[int] = list(range(num_slots - 1, -1, -1))
+
+    @property
+    def free_slots(self) -> int:
+        return len(self._free)
+
+    def alloc(self) -> int:
+        if not self._free:
+            raise OutOfSlots(f"all {self.num_slots} state slots are in use")
+        return self._free.pop()
+
+    def free(self, slot: int) -> None:
+        self._free.append(slot)
+
+
 @dataclass
 class Session:
     """One persistent conversation's KV state for one hosted model."""
     session_id: str
     token_ids: List[int] = field(default_factory=list)   # tokens whose KV is cached
     blocks: List[int] = field(default_factory=list)
+    state_slot: int = -1                # recurrent state, -1: none held
 
     def slot(self, pos: int, block_size: int) -> int:
         return self.blocks[pos // block_size] * block_size + pos % block_size
@@ -58,8 +87,10 @@ class Session:
 class SessionCache:
     """session_id -> Session with LRU eviction under block pressure."""
 
-    def __init__(self, mgr: BlockManager):
+    def __init__(self, mgr: BlockManager,
+                 states: Optional[StateSlots] = None):
         self.mgr = mgr
+        self.states = states            # None: no recurrent state
         self._sessions: Dict[str, Session] = {}
         self._lru: List[str] = []
 
@@ -82,16 +113,23 @@ class SessionCache:
             self.mgr.free(sess.blocks)
             sess.blocks = []
             sess.token_ids = []
+            if sess.state_slot >= 0:
+                self.states.free(sess.state_slot)
+                sess.state_slot = -1
         if session_id in self._lru:
             self._lru.remove(session_id)
 
     def match_prefix(self, sess: Session, prompt: List[int]) -> int:
         """Longest common prefix of the cached tokens and the new prompt;
-        trailing cached tokens (a diverged tail) are discarded."""
+        trailing cached tokens (a diverged tail) are discarded.  The prompt's
+        last token is never taken from the cache: its logits are needed.
+        With a recurrent state it is the whole cached sequence or nothing."""
         n = 0
-        limit = min(len(sess.token_ids), len(prompt))
+        limit = min(len(sess.token_ids), len(prompt) - 1)
         while n < limit and sess.token_ids[n] == prompt[n]:
             n += 1
+        if self.states is not None and n < len(sess.token_ids):
+            n = 0
         if n < len(sess.token_ids):
             keep_blocks = self.mgr.blocks_for_tokens(n)
             self.mgr.free(sess.blocks[keep_blocks:])
@@ -99,23 +137,44 @@ class SessionCache:
             sess.token_ids = sess.token_ids[:n]
         return n
 
+    def _evict(self, sess: Session, active: Optional[List[str]]) -> bool:
+        """Drop the least recently used idle session, if there is one."""
+        victim = next((sid for sid in self._lru
+                       if sid != sess.session_id
+                       and (active is None or sid not in active)), None)
+        if victim is None:
+            return False
+        self.drop(victim)
+        return True
+
+    def place(self, sess: Session,
+              active: Optional[List[str]] = None) -> bool:
+        """Give the session a state slot (evicting idle LRU sessions); False:
+        all slots are held by active sessions, try again later."""
+        if self.states is None or sess.state_slot >= 0:
+            return True
+        while not self.states.free_slots:
+            if not self._evict(sess, active):
+                return False
+        sess.state_slot = self.states.alloc()
+        return True
+
     def extend(self, sess: Session, new_tokens: List[int],
                active: Optional[List[str]] = None) -> List[int]:
         """Allocate blocks for new tokens (evicting idle LRU sessions under
         pressure) and record them; returns the global slots."""
+        if not self.place(sess, active):
+            raise OutOfSlots(f"all {self.states.num_slots} state slots are "
+                             f"held by active sequences")
         bs = self.mgr.block_size
         start = len(sess.token_ids)
         need_blocks = self.mgr.blocks_for_tokens(start + len(new_tokens)) \
             - len(sess.blocks)
         while need_blocks > self.mgr.free_blocks:
-            victim = next((sid for sid in self._lru
-                           if sid != sess.session_id
-                           and (active is None or sid not in active)), None)
-            if victim is None:
+            if not self._evict(sess, active):
                 raise OutOfBlocks(
                     f"KV pool exhausted: need {need_blocks} blocks, "
                     f"{self.mgr.free_blocks} free, no evictable session")
-            self.drop(victim)
         if need_blocks > 0:
             sess.blocks.extend(self.mgr.alloc(need_blocks))
         sess.token_ids.extend(new_tokens)

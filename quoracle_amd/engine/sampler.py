@@ -398,6 +398,9 @@ class Sampler:
                 sub = sub + mask
             probs = torch.softmax(sub / temps, dim=-1)
             for i, r in enumerate(rows):
+                if params[r].temperature <= 0.0:        # greedy
+                    pending.append((r, sub[i].argmax().view(1)))
+                    continue
                 row_probs = probs[i]
                 if params[r].top_p < 1.0:
                     row_probs = _top_p_filter(row_probs, params[r].top_p)

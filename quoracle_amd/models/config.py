@@ -1,16 +1,24 @@
-"""Model architecture configs (Llama-family + MoE) for the local pool.
+"""Model registry: architecture configs (Llama-family, MoE, hybrid) for the
+local pool.
 
 The reference delegates model choice to remote providers (reference:
 lib/quoracle/models/model_query.ex); here each pool entry names a locally
 hosted architecture.  A model key is "<preset>#<instance>" — instances share
 the architecture but get different random-init seeds, giving the consensus
-pool genuinely decorrelated voters.
+pool genuinely decorrelated voters.  A key may also be "<folder>" or
+"<folder>#<instance>": a checkpoint folder with config.json and
+model.safetensors, whose "architecture" names the config and model class.
 """
 
 from __future__ import annotations
 
+import functools
+import json
+import os
 from dataclasses import dataclass
-from typing import Dict
+from typing import Dict, Union
+
+from .hybrid_config import KoridraConfig, koridra_preset
 
 
 @dataclass(frozen=True)
@@ -32,6 +40,11 @@ class ModelConfig:
     n_experts: int = 0
     top_k_experts: int = 2
 
+    architecture = "Llama"
+    native_module = "_quoracle_ops"
+    is_hybrid = False
+    needs_state = False         # no recurrent state beside the KV pages
+
     @property
     def q_dim(self) -> int:
         return self.n_heads * self.head_dim
@@ -48,9 +61,9 @@ class ModelConfig:
     def is_moe(self) -> bool:
         return self.n_experts > 0
 
-    def kv_bytes_per_token(self) -> int:
-        """bf16 paged-KV footprint of one token across all layers."""
-        return 2 * 2 * self.n_layers * self.kv_dim
+    def kv_bytes_per_token(self, element: int = 2) -> int:
+        """Paged-KV footprint of one token across all layers."""
+        return 2 * element * self.n_layers * self.kv_dim
 
     def param_count(self) -> int:
         embed = self.vocab_size * self.hidden
@@ -65,7 +78,9 @@ class ModelConfig:
         return embed + lm_head + self.n_layers * per_layer + self.hidden
 
 
-PRESETS: Dict[str, ModelConfig] = {
+AnyConfig = Union[ModelConfig, KoridraConfig]
+
+PRESETS: Dict[str, AnyConfig] = {
     # CPU-testable toy model (head_dim multiple of 8, <=128 for the kernels)
     "tiny": ModelConfig("tiny", vocab_size=512, n_layers=2, hidden=64,
                         n_heads=4, n_kv_heads=2, head_dim=16,
@@ -110,16 +125,49 @@ PRESETS: Dict[str, ModelConfig] = {
                                head_dim=64, intermediate=512,
                                rope_theta=10000.0, max_context=4096,
                                max_output=1, tie_embeddings=True),
+    # CPU-testable Koridra toy
+    "koridra-tiny": koridra_preset(
+        "koridra-tiny", vocab=512, hidden=64, n_layers=4, ff=96, heads=4,
+        kv_heads=2, dim=16, chunk=48, lin_heads=2, lin_dim=16, lin_vdim=24,
+        max_context=4096, every=2, max_output=1024, base=10000.0, rank=4),
+    # Koridra with the layer sizes of a 1B-class and of an 8B-class model
+    "koridra-1b": koridra_preset(
+        "koridra-1b", vocab=128256, hidden=2048, n_layers=16, ff=8192,
+        heads=16, kv_heads=4, dim=128, chunk=4096, lin_heads=16, lin_dim=128,
+        lin_vdim=128, max_context=32768),
+    "koridra-8b": koridra_preset(
+        "koridra-8b", vocab=128256, hidden=4096, n_layers=32, ff=14336,
+        heads=32, kv_heads=8, dim=128, chunk=8192, lin_heads=32, lin_dim=128,
+        lin_vdim=128, max_context=32768),
 }
 
+# config.json "architecture" -> reader of the rest of the file
+ARCHITECTURES = {"Koridra": KoridraConfig.from_dict}
 
-def get_config(key: str) -> ModelConfig:
-    """Resolve "<preset>#<instance>" or "<preset>" to its architecture."""
+
+@functools.lru_cache(maxsize=64)
+def load_config(folder: str) -> AnyConfig:
+    """The config of a checkpoint folder, by its config.json."""
+    with open(os.path.join(folder, "config.json")) as f:
+        raw = json.load(f)
+    arch = raw.get("architecture")
+    if arch not in ARCHITECTURES:
+        raise KeyError(f"{folder}: unknown architecture {arch!r} "
+                       f"(known: {sorted(ARCHITECTURES)})")
+    name = os.path.basename(os.path.abspath(folder))
+    return ARCHITECTURES[arch](raw, name=name, path=folder)
+
+
+def get_config(key: str) -> AnyConfig:
+    """Resolve "<preset>#<instance>", "<preset>" or a checkpoint folder to
+    its architecture."""
     preset = key.split("#", 1)[0]
-    if preset not in PRESETS:
-        raise KeyError(f"unknown model preset {preset!r} "
-                       f"(known: {sorted(PRESETS)})")
-    return PRESETS[preset]
+    if preset in PRESETS:
+        return PRESETS[preset]
+    if os.path.isfile(os.path.join(preset, "config.json")):
+        return load_config(preset)
+    raise KeyError(f"unknown model preset {preset!r} "
+                   f"(known: {sorted(PRESETS)}, or a checkpoint folder)")
 
 
 def instance_seed(key: str) -> int:

@@ -58,10 +58,33 @@ class ForwardBatch:
     tile32_seq: Optional[torch.Tensor] = None
     tile32_pos0: Optional[torch.Tensor] = None
     sample_rows: Optional[torch.Tensor] = None  # [R] int64 rows needing logits
+    # -- hybrid models (recurrent state beside the KV pages) ----------------
+    row_seq: Optional[torch.Tensor] = None    # [T] row into block_tables
+    state_slots: Optional[torch.Tensor] = None  # [B_all] state slot per seq
+    # prefill sequences (block_tables rows n_decode..) and their
+    # linear-attention chunks: rows, lengths, chunks seg_chunk0[i]..[i+1]
+    seg_row0: Optional[torch.Tensor] = None
+    seg_len: Optional[torch.Tensor] = None
+    seg_chunk0: Optional[torch.Tensor] = None   # [n_prefill + 1]
+    chunk_row0: Optional[torch.Tensor] = None
+    chunk_len: Optional[torch.Tensor] = None
 
     @property
     def total_tokens(self) -> int:
         return self.tokens.shape[0]
+
+    def hybrid_tensors(self) -> Dict[str, torch.Tensor]:
+        """What the hybrid forward driver reads, by its names."""
+        named = {
+            "tokens": self.tokens, "positions": self.positions,
+            "slots": self.slots, "block_tables": self.block_tables,
+            "ctx_lens": self.ctx_lens, "row_seq": self.row_seq,
+            "tile_q0": self.tile32_q0, "tile_qn": self.tile32_qn,
+            "tile_seq": self.tile32_seq, "tile_pos0": self.tile32_pos0,
+            "state_slots": self.state_slots, "seg_row0": self.seg_row0,
+            "seg_len": self.seg_len, "seg_chunk0": self.seg_chunk0,
+            "chunk_row0": self.chunk_row0, "chunk_len": self.chunk_len}
+        return {k: t for k, t in named.items() if t is not None}
 
 
 class KVCache:
@@ -76,6 +99,11 @@ class KVCache:
                   for _ in range(cfg.n_layers)]
         self.v = [torch.zeros(shape, dtype=torch.bfloat16, device=device)
                   for _ in range(cfg.n_layers)]
+        self.state_slots = 0
+
+    def clear(self) -> None:
+        for t in self.k + self.v:
+            t.zero_()
 
     def bytes(self) -> int:
         return sum(t.numel() * 2 for t in self.k) * 2
@@ -203,7 +231,8 @@ class LlamaModel:
             n += sum(t.numel() for t in layer.values())
         return n * self.embed.element_size()
 
-    def new_kv_cache(self, num_blocks: int, block_size: int) -> KVCache:
+    def new_kv_cache(self, num_blocks: int, block_size: int,
+                     state_slots: int = 0) -> KVCache:
         return KVCache(self.lcfg, num_blocks, block_size, self.device)
 
     # -- forward -------------------------------------------------------------

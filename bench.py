@@ -55,6 +55,12 @@ def parse_args():
                         "lockstep TP group hosting a '+'-joined model pool "
                         "(BASELINE config 5: --tp 4 --model "
                         "llama3-70b+mixtral-8x7b)")
+    p.add_argument("--layer-bench", action="store_true",
+                   help="instead of the flagship workload: prefill and "
+                        "decode throughput of Koridra layers beside Llama "
+                        "layers of equal size, one JSON line each")
+    p.add_argument("--layer-bench-only", choices=["koridra", "llama"],
+                   default=None, help="one side of --layer-bench (profiling)")
     return p.parse_args()
 
 
@@ -74,6 +80,10 @@ def main():
     import torch
     print(f"[bench t={time.perf_counter() - T_START:.1f}s] torch imported",
           file=sys.stderr, flush=True)
+    if args.layer_bench:
+        from quoracle_amd.tools import layer_bench
+        layer_bench.main(device=args.device, only=args.layer_bench_only)
+        return
 
     rank = int(os.environ.get("RANK", "0"))
     world = int(os.environ.get("WORLD_SIZE", "1"))

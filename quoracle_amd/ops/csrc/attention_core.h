@@ -39,23 +39,16 @@ __device__ __forceinline__ int swz(int row, int d) {
   return d ^ (((row >> 1) & 7) << 3);
 }
 
-__device__ __forceinline__ unsigned int pack_pair(float lo, float hi) {
-  union { bf16 h; unsigned short u; } a, b;
-  a.h = f2bf(lo);
-  b.h = f2bf(hi);
-  return (unsigned int)a.u | ((unsigned int)b.u << 16);
-}
-
 // Two C-layout key blocks of a transposed score tile (lane: query row =
 // lane&15, keys (lane>>4)*4 + reg of each block) -> the A fragment of those
 // 32 keys (lane: row = lane&15, keys (lane>>4)*8 + i): pack to bf16 dwords,
 // then a permlane32 + permlane16 swap pair.
 __device__ __forceinline__ bf16x8_t scores_to_afrag(const f32x4_t &s0,
                                                     const f32x4_t &s1) {
-  unsigned int d0 = pack_pair(s0[0], s0[1]);
-  unsigned int d1 = pack_pair(s0[2], s0[3]);
-  unsigned int e0 = pack_pair(s1[0], s1[1]);
-  unsigned int e1 = pack_pair(s1[2], s1[3]);
+  unsigned int d0 = pack_bf16x2(s0[0], s0[1]);
+  unsigned int d1 = pack_bf16x2(s0[2], s0[3]);
+  unsigned int e0 = pack_bf16x2(s1[0], s1[1]);
+  unsigned int e1 = pack_bf16x2(s1[2], s1[3]);
   {
     auto r = __builtin_amdgcn_permlane32_swap(d0, e0, false, false);
     d0 = r[0]; e0 = r[1];

@@ -24,11 +24,12 @@ __device__ __forceinline__ void unpack_bf16x2(unsigned int u, float &lo, float &
   hi = __bfloat162float(*reinterpret_cast<__hip_bfloat16 *>(&b));
 }
 
+// Two floats rounded to nearest even, one conversion instruction.
 __device__ __forceinline__ unsigned int pack_bf16x2(float lo, float hi) {
-  bf16 a = f2bf(lo), b = f2bf(hi);
-  unsigned short ua = *reinterpret_cast<unsigned short *>(&a);
-  unsigned short ub = *reinterpret_cast<unsigned short *>(&b);
-  return (unsigned int)ua | ((unsigned int)ub << 16);
+  typedef float f32x2 __attribute__((ext_vector_type(2)));
+  typedef __bf16 b16x2 __attribute__((ext_vector_type(2)));
+  const f32x2 v = {lo, hi};
+  return __builtin_bit_cast(unsigned int, __builtin_convertvector(v, b16x2));
 }
 
 // Wave-wide (64-lane) sum/max via xor shuffles.

@@ -53,9 +53,18 @@ template <typename F> void by_dtype(const Tensor &t, F body) {
   else if (t.scalar_type() == torch::kFloat32) body(float());
   else TORCH_CHECK(false, "activations must be bfloat16 or float32");
 }
-template <typename F> void by_vec(bool vec4, F body) {
-  if (vec4) body(std::integral_constant<int, 4>());
-  else body(std::integral_constant<int, 1>());
+template <int N> using Int = std::integral_constant<int, N>;
+template <typename F> void by_vec(bool vec8, F body) {
+  if (vec8) body(Int<8>());
+  else body(Int<1>());
+}
+// Register groups per thread of a 256-thread norm over n values; 0: too many.
+template <typename F> void by_items(int n, int vec, F body) {
+  const int need = (n + 256 * vec - 1) / (256 * vec);
+  if (need <= 1) body(Int<1>());
+  else if (need <= 2) body(Int<2>());
+  else if (need <= 4) body(Int<4>());
+  else body(Int<0>());
 }
 
 void embed_positions(Tensor x, Tensor h, Tensor embed, OptTensor table,
@@ -70,7 +79,7 @@ void embed_positions(Tensor x, Tensor h, Tensor embed, OptTensor table,
   if (T == 0) return;
   by_dtype(embed, [&](auto t0) {
     using A = decltype(t0);
-    by_vec(n % 4 == 0, [&](auto v) {
+    by_vec(n % 8 == 0, [&](auto v) {
       embed_positions_kernel<A, decltype(v)::value>
           <<<dim3(T), dim3(256), 0, current_stream()>>>(
               fptr(x), ptr<A>(h), ptr<A>(embed),
@@ -92,12 +101,14 @@ void post_norm(Tensor x, Tensor h, Tensor a, double sa, OptTensor b,
   if (T == 0) return;
   by_dtype(h, [&](auto t0) {
     using A = decltype(t0);
-    by_vec(n % 4 == 0, [&](auto v) {
-      post_norm_kernel<A, decltype(v)::value>
-          <<<dim3(T), dim3(256), 0, current_stream()>>>(
-              fptr(x), ptr<A>(h), ptr<A>(a), (float)sa,
-              b ? ptr<A>(*b) : nullptr, (float)sb, (float)alpha, fptr(w), n,
-              (float)eps);
+    by_vec(n % 8 == 0, [&](auto v) {
+      by_items(n, v, [&](auto ni) {
+        post_norm_kernel<A, decltype(v)::value, decltype(ni)::value>
+            <<<dim3(T), dim3(256), 0, current_stream()>>>(
+                fptr(x), ptr<A>(h), ptr<A>(a), (float)sa,
+                b ? ptr<A>(*b) : nullptr, (float)sb, (float)alpha, fptr(w), n,
+                (float)eps);
+      });
     });
   });
   HIP_CHECK_KERNEL();
@@ -112,7 +123,7 @@ void norm_rows(Tensor out, Tensor x, Tensor rows, Tensor w, double eps) {
   if (R == 0) return;
   by_dtype(out, [&](auto t0) {
     using A = decltype(t0);
-    by_vec(n % 4 == 0, [&](auto v) {
+    by_vec(n % 8 == 0, [&](auto v) {
       norm_rows_kernel<A, decltype(v)::value>
           <<<dim3(R), dim3(256), 0, current_stream()>>>(
               ptr<A>(out), fptr(x),
@@ -131,7 +142,7 @@ void glu(Tensor out, Tensor gu) {
   if (T == 0) return;
   by_dtype(out, [&](auto t0) {
     using A = decltype(t0);
-    by_vec(n % 4 == 0, [&](auto v) {
+    by_vec(n % 8 == 0, [&](auto v) {
       constexpr int VEC = decltype(v)::value;
       glu_kernel<A, VEC>
           <<<dim3(T, (n + 256 * VEC - 1) / (256 * VEC)), dim3(256), 0,
@@ -150,16 +161,29 @@ void gated_norm(Tensor out, Tensor o, Tensor proj, int64_t g_off, Tensor w,
               "gated_norm shapes");
   TORCH_CHECK(g_off + groups * n <= stride, "gated_norm gate");
   if (T == 0) return;
-  const bool vec = n % 4 == 0 && stride % 4 == 0 && g_off % 4 == 0;
-  const int per = vec ? n / 4 : n;
-  const int block = per <= 64 ? 64 : per <= 128 ? 128 : 256;
+  const bool vec = n % 8 == 0 && stride % 8 == 0 && g_off % 8 == 0;
   by_dtype(out, [&](auto t0) {
     using A = decltype(t0);
     by_vec(vec, [&](auto v) {
-      gated_norm_kernel<A, decltype(v)::value>
-          <<<dim3(T, groups), dim3(block), 0, current_stream()>>>(
-              ptr<A>(out), ptr<A>(o), ptr<A>(proj), stride, (int)g_off,
-              fptr(w), n, (int)act, (float)eps);
+      constexpr int VEC = decltype(v)::value;
+      auto small = [&](auto lpg) {
+        constexpr int LPG = decltype(lpg)::value;
+        gated_norm_small_kernel<A, VEC, LPG>
+            <<<dim3((T * groups * LPG + 255) / 256), dim3(256), 0,
+               current_stream()>>>(
+                ptr<A>(out), ptr<A>(o), ptr<A>(proj), stride, (int)g_off,
+                fptr(w), n, (int)groups, T * groups, (int)act, (float)eps);
+      };
+      if (n <= 8 * VEC) small(Int<8>());
+      else if (n <= 16 * VEC) small(Int<16>());
+      else if (n <= 64 * VEC) small(Int<64>());
+      else
+        by_items(n, v, [&](auto ni) {
+          gated_norm_kernel<A, VEC, decltype(ni)::value>
+              <<<dim3(T, groups), dim3(256), 0, current_stream()>>>(
+                  ptr<A>(out), ptr<A>(o), ptr<A>(proj), stride, (int)g_off,
+                  fptr(w), n, (int)act, (float)eps);
+        });
     });
   });
   HIP_CHECK_KERNEL();
@@ -216,12 +240,17 @@ void log_decay(Tensor out, Tensor proj, int64_t a_off, Tensor a2, Tensor bias,
   if (runs == 0) return;
   by_dtype(proj, [&](auto t0) {
     using A = decltype(t0);
-    log_decay_kernel<A>
-        <<<dim3(runs, (C + 255) / 256), dim3(256), 0, current_stream()>>>(
-            fptr(out) + first * C, ptr<A>(proj) + first * stride, stride,
-            (int)a_off, rank, ptr<A>(a2), fptr(bias), (float)(1.0 / tau), C,
-            run_row0 ? iptr(*run_row0) : nullptr,
-            run_row0 ? iptr(*run_len) : nullptr);
+    auto run = [&](auto rmax) {
+      log_decay_kernel<A, decltype(rmax)::value>
+          <<<dim3(runs, (C + 255) / 256), dim3(256), 0, current_stream()>>>(
+              fptr(out) + first * C, ptr<A>(proj) + first * stride, stride,
+              (int)a_off, rank, ptr<A>(a2), fptr(bias), (float)(1.0 / tau),
+              C, run_row0 ? iptr(*run_row0) : nullptr,
+              run_row0 ? iptr(*run_len) : nullptr);
+    };
+    if (rank <= 16) run(Int<16>());
+    else if (rank <= 64) run(Int<64>());
+    else run(Int<0>());
   });
   HIP_CHECK_KERNEL();
 }
@@ -284,7 +313,7 @@ void local_attn_prefill(Tensor out, Tensor q, Tensor kc, Tensor vc, Tensor bt,
   if (chunk > 0) seen = std::min<long>(seen, chunk + 127);
   long ns = 1;
   if (seen >= 1024)
-    ns = std::max<long>(1, std::min<long>({16, 1024 / (nt * a.Hq),
+    ns = std::max<long>(1, std::min<long>({16, 512 / (nt * a.Hq),
                                            seen / 256}));
   Tensor pm, pl, pa;
   if (ns > 1) {
@@ -456,17 +485,29 @@ void linear_chunked(Tensor o, Tensor proj, int64_t q_off, int64_t k_off,
   auto ws = torch::empty({nc, a.H, a.V, a.D},
                          proj.options().dtype(torch::kFloat32));
   auto stream = current_stream();
-  const int tiles = ((a.D + 63) / 64) * ((a.V + 63) / 64);
+  const Tensor state_pool = state;
   const dim3 g_scan(ns, a.H, (a.V * a.D + 1023) / 1024);
   auto run = [&](auto ch_, auto nk_) {
     constexpr bool CH = decltype(ch_)::value;
-    linear_chunk_state_kernel<CH>
-        <<<dim3(nc, a.H, tiles), dim3(256), 0, stream>>>(
-            fptr(ws), ptr<bf16>(proj), a.stride, a.k_off, a.v_off, a.H, a.D,
-            a.V, (int)act, fptr(decay), iptr(chunk_row0), iptr(chunk_len));
+    auto state = [&](auto td_, auto tv_) {
+      constexpr int TD = decltype(td_)::value, TV = decltype(tv_)::value;
+      const int tiles = ((a.D + TD - 1) / TD) * ((a.V + TV - 1) / TV);
+      linear_chunk_state_kernel<CH, TD, TV>
+          <<<dim3(nc, a.H, tiles), dim3(256), 0, stream>>>(
+              fptr(ws), ptr<bf16>(proj), a.stride, a.k_off, a.v_off, a.H,
+              a.D, a.V, (int)act, fptr(decay), iptr(chunk_row0),
+              iptr(chunk_len));
+    };
+    if (a.D <= 64) {
+      if (a.V <= 64) state(Int<64>(), Int<64>());
+      else state(Int<64>(), Int<128>());
+    } else {
+      if (a.V <= 64) state(Int<128>(), Int<64>());
+      else state(Int<128>(), Int<128>());
+    }
     HIP_CHECK_KERNEL();
     linear_chunk_scan_kernel<CH><<<g_scan, dim3(256), 0, stream>>>(
-        fptr(ws), fptr(state), a.H, a.D, a.V, fptr(decay), iptr(chunk_row0),
+        fptr(ws), fptr(state_pool), a.H, a.D, a.V, fptr(decay), iptr(chunk_row0),
         iptr(chunk_len), iptr(seg_row0), iptr(seg_chunk0), iptr(seg_slot),
         iptr(positions));
     HIP_CHECK_KERNEL();

@@ -2,7 +2,9 @@
 // models.  T is the activation type (bf16 or float); the residual stream, all
 // norms, gates of a recurrence and position angles are float32.
 //
-// VEC = 4 kernels need every row start to be a multiple of 4 elements.
+// VEC > 1 kernels need every row start to be a multiple of VEC elements.
+// Norm kernels keep their row in registers: NI groups of VEC per thread.
+// NI = 0 (rows that do not fit) reads the row a second time instead.
 
 #include "hybrid_common.h"
 
@@ -37,7 +39,7 @@ embed_positions_kernel(float *__restrict__ x, T *__restrict__ h,
 // Norm after the sum: x <- rms(alpha*x + sa*a (+ sb*b)) * w in place;
 // h = T(x).  Grid: (T); block 256.
 // ---------------------------------------------------------------------------
-template <typename T, int VEC>
+template <typename T, int VEC, int NI>
 __global__ void __launch_bounds__(256)
 post_norm_kernel(float *__restrict__ x, T *__restrict__ h,
                  const T *__restrict__ a, float sa, const T *__restrict__ b,
@@ -45,32 +47,56 @@ post_norm_kernel(float *__restrict__ x, T *__restrict__ h,
                  float eps) {
   __shared__ float scratch[4];
   const long row = (long)blockIdx.x * n;
-  float ssq = 0.f;
-  for (int i = threadIdx.x * VEC; i < n; i += 256 * VEC) {
-    float xv[VEC], av[VEC], bv[VEC];
+  auto sum_at = [&](int i, float *xv) {
+    float av[VEC];
     hyb::load_v<VEC>(x + row + i, xv);
     hyb::load_v<VEC>(a + row + i, av);
 #pragma unroll
     for (int k = 0; k < VEC; ++k) xv[k] = alpha * xv[k] + sa * av[k];
     if (b) {
-      hyb::load_v<VEC>(b + row + i, bv);
+      hyb::load_v<VEC>(b + row + i, av);
 #pragma unroll
-      for (int k = 0; k < VEC; ++k) xv[k] += sb * bv[k];
+      for (int k = 0; k < VEC; ++k) xv[k] += sb * av[k];
     }
-#pragma unroll
-    for (int k = 0; k < VEC; ++k) ssq += xv[k] * xv[k];
-    hyb::store_v<VEC>(x + row + i, xv);
-  }
-  const float inv = 1.f / sqrtf(block_sum(ssq, scratch) / (float)n + eps);
-  // each thread re-reads only what it wrote itself
-  for (int i = threadIdx.x * VEC; i < n; i += 256 * VEC) {
-    float xv[VEC], wv[VEC];
-    hyb::load_v<VEC>(x + row + i, xv);
+  };
+  auto finish = [&](int i, float *xv, float inv) {
+    float wv[VEC];
     hyb::load_v<VEC>(w + i, wv);
 #pragma unroll
     for (int k = 0; k < VEC; ++k) xv[k] = xv[k] * inv * wv[k];
     hyb::store_v<VEC>(x + row + i, xv);
     hyb::store_v<VEC>(h + row + i, xv);
+  };
+  float ssq = 0.f;
+  if constexpr (NI > 0) {
+    float v[NI][VEC];
+#pragma unroll
+    for (int it = 0; it < NI; ++it) {
+      const int i = (it * 256 + threadIdx.x) * VEC;
+      if (i >= n) continue;
+      sum_at(i, v[it]);
+#pragma unroll
+      for (int k = 0; k < VEC; ++k) ssq += v[it][k] * v[it][k];
+    }
+    const float inv = 1.f / sqrtf(block_sum(ssq, scratch) / (float)n + eps);
+#pragma unroll
+    for (int it = 0; it < NI; ++it) {
+      const int i = (it * 256 + threadIdx.x) * VEC;
+      if (i < n) finish(i, v[it], inv);
+    }
+  } else {
+    for (int i = threadIdx.x * VEC; i < n; i += 256 * VEC) {
+      float v[VEC];
+      sum_at(i, v);
+#pragma unroll
+      for (int k = 0; k < VEC; ++k) ssq += v[k] * v[k];
+    }
+    const float inv = 1.f / sqrtf(block_sum(ssq, scratch) / (float)n + eps);
+    for (int i = threadIdx.x * VEC; i < n; i += 256 * VEC) {
+      float v[VEC];
+      sum_at(i, v);
+      finish(i, v, inv);
+    }
   }
 }
 
@@ -117,16 +143,16 @@ glu_kernel(T *__restrict__ out, const T *__restrict__ gu, int n) {
   hyb::load_v<VEC>(gu + t * 2 * n + i, g);
   hyb::load_v<VEC>(gu + t * 2 * n + n + i, u);
 #pragma unroll
-  for (int k = 0; k < VEC; ++k) g[k] = g[k] * hyb::sigmoid_f(g[k]) * u[k];
+  for (int k = 0; k < VEC; ++k) g[k] = g[k] * hyb::sigmoid_t<T>(g[k]) * u[k];
   hyb::store_v<VEC>(out + t * n + i, g);
 }
 
 // ---------------------------------------------------------------------------
 // Norm each group of `n` values of o[t] (a head, or all heads together),
 // times w[n], times act(gate): out[t, g*n + i].  The gate is read in place
-// from the fused projection row.  Grid: (T, groups); block = multiple of 64.
+// from the fused projection row.  Grid: (T, groups); block 256.
 // ---------------------------------------------------------------------------
-template <typename T, int VEC>
+template <typename T, int VEC, int NI>
 __global__ void __launch_bounds__(256)
 gated_norm_kernel(T *__restrict__ out, const T *__restrict__ o,
                   const T *__restrict__ proj, long stride, int g_off,
@@ -135,25 +161,78 @@ gated_norm_kernel(T *__restrict__ out, const T *__restrict__ o,
   const long t = blockIdx.x;
   const long base = (t * gridDim.y + blockIdx.y) * (long)n;
   const T *gate = proj + t * stride + g_off + (long)blockIdx.y * n;
-  const int step = blockDim.x * VEC;
-  float ssq = 0.f;
-  for (int i = threadIdx.x * VEC; i < n; i += step) {
-    float v[VEC];
-    hyb::load_v<VEC>(o + base + i, v);
-#pragma unroll
-    for (int k = 0; k < VEC; ++k) ssq += v[k] * v[k];
-  }
-  const float inv = 1.f / sqrtf(block_sum(ssq, scratch) / (float)n + eps);
-  for (int i = threadIdx.x * VEC; i < n; i += step) {
-    float v[VEC], gv[VEC], wv[VEC];
-    hyb::load_v<VEC>(o + base + i, v);
+  auto finish = [&](int i, float *v, float inv) {
+    float gv[VEC], wv[VEC];
     hyb::load_v<VEC>(gate + i, gv);
     hyb::load_v<VEC>(w + i, wv);
 #pragma unroll
     for (int k = 0; k < VEC; ++k)
-      v[k] = v[k] * inv * wv[k] * hyb::activate(gv[k], act);
+      v[k] = v[k] * inv * wv[k] * hyb::activate<T>(gv[k], act);
     hyb::store_v<VEC>(out + base + i, v);
+  };
+  float ssq = 0.f;
+  if constexpr (NI > 0) {
+    float v[NI][VEC];
+#pragma unroll
+    for (int it = 0; it < NI; ++it) {
+      const int i = (it * 256 + threadIdx.x) * VEC;
+      if (i >= n) continue;
+      hyb::load_v<VEC>(o + base + i, v[it]);
+#pragma unroll
+      for (int k = 0; k < VEC; ++k) ssq += v[it][k] * v[it][k];
+    }
+    const float inv = 1.f / sqrtf(block_sum(ssq, scratch) / (float)n + eps);
+#pragma unroll
+    for (int it = 0; it < NI; ++it) {
+      const int i = (it * 256 + threadIdx.x) * VEC;
+      if (i < n) finish(i, v[it], inv);
+    }
+  } else {
+    for (int i = threadIdx.x * VEC; i < n; i += 256 * VEC) {
+      float v[VEC];
+      hyb::load_v<VEC>(o + base + i, v);
+#pragma unroll
+      for (int k = 0; k < VEC; ++k) ssq += v[k] * v[k];
+    }
+    const float inv = 1.f / sqrtf(block_sum(ssq, scratch) / (float)n + eps);
+    for (int i = threadIdx.x * VEC; i < n; i += 256 * VEC) {
+      float v[VEC];
+      hyb::load_v<VEC>(o + base + i, v);
+      finish(i, v, inv);
+    }
   }
+}
+
+// The same for groups of at most LPG*VEC values: LPG lanes per group, many
+// groups per workgroup.  Grid: ceil(T*groups*LPG / 256); block 256.
+template <typename T, int VEC, int LPG>
+__global__ void __launch_bounds__(256)
+gated_norm_small_kernel(T *__restrict__ out, const T *__restrict__ o,
+                        const T *__restrict__ proj, long stride, int g_off,
+                        const float *__restrict__ w, int n, int groups,
+                        long total, int act, float eps) {
+  const long at = ((long)blockIdx.x * 256 + threadIdx.x) / LPG;
+  const int i = (threadIdx.x % LPG) * VEC;
+  const bool live = at < total && i < n;
+  float v[VEC];
+  float ssq = 0.f;
+  if (live) {
+    hyb::load_v<VEC>(o + at * n + i, v);
+#pragma unroll
+    for (int k = 0; k < VEC; ++k) ssq += v[k] * v[k];
+  }
+#pragma unroll
+  for (int s = LPG / 2; s >= 1; s >>= 1) ssq += __shfl_xor(ssq, s, LPG);
+  if (!live) return;
+  const float inv = 1.f / sqrtf(ssq / (float)n + eps);
+  float gv[VEC], wv[VEC];
+  hyb::load_v<VEC>(proj + at / groups * stride + g_off + at % groups * n + i,
+                   gv);
+  hyb::load_v<VEC>(w + i, wv);
+#pragma unroll
+  for (int k = 0; k < VEC; ++k)
+    v[k] = v[k] * inv * wv[k] * hyb::activate<T>(gv[k], act);
+  hyb::store_v<VEC>(out + at * n + i, v);
 }
 
 // ---------------------------------------------------------------------------
@@ -250,34 +329,57 @@ qk_norm_rope_store_kernel(
 // run_row0 null: every row is a run of its own (out = ld).
 // Grid: (runs, ceil(C/256)); block 256, one channel per thread.
 // ---------------------------------------------------------------------------
-template <typename T>
+// RMAX: rank the channel's weights are held in registers for; 0: any rank.
+template <typename T, int RMAX>
 __global__ void __launch_bounds__(256)
 log_decay_kernel(float *__restrict__ out, const T *__restrict__ proj,
                  long stride, int a_off, int rank, const T *__restrict__ a2,
                  const float *__restrict__ bias, float inv_tau, int C,
                  const int *__restrict__ run_row0,
                  const int *__restrict__ run_len) {
-  const int c = blockIdx.y * 256 + threadIdx.x;
-  if (c >= C) return;
+  constexpr int TB = 64;                       // rows staged at a time
+  constexpr int RS = RMAX ? RMAX : 1;
+  __shared__ __align__(16) float a_s[TB * RS];
+  const int c = min((int)(blockIdx.y * 256 + threadIdx.x), C - 1);
+  const bool live = blockIdx.y * 256 + threadIdx.x < C;
   const long row0 = run_row0 ? run_row0[blockIdx.x] : (int)blockIdx.x;
   const int len = run_row0 ? run_len[blockIdx.x] : 1;
   const T *wr = a2 + (long)c * rank;
-  float w[16];
-#pragma unroll
-  for (int r = 0; r < 16; ++r) w[r] = r < rank ? hyb::to_f(wr[r]) : 0.f;
   const float b = bias[c];
-  float sum = 0.f;
-  for (int t = 0; t < len; ++t) {
-    const T *a = proj + (row0 + t) * stride + a_off;
-    float z = 0.f;
+  float w[RS];
 #pragma unroll
-    for (int r = 0; r < 16; ++r)
-      if (r < rank) z = fmaf(w[r], hyb::to_f(a[r]), z);
-    for (int r = 16; r < rank; ++r)
-      z = fmaf(hyb::to_f(wr[r]), hyb::to_f(a[r]), z);
-    z += b;
+  for (int r = 0; r < RS; ++r) w[r] = r < rank ? hyb::to_f(wr[r]) : 0.f;
+  float sum = 0.f;
+  auto put_row = [&](int t, float z) {
     const float ls = fminf(z, 0.f) - log1pf(expf(-fabsf(z)));
     sum += ls * inv_tau;
-    out[(row0 + t) * (long)C + c] = sum;
+    if (live) out[(row0 + t) * (long)C + c] = sum;
+  };
+  if constexpr (RMAX > 0) {
+    for (int t0 = 0; t0 < len; t0 += TB) {
+      const int tn = min(TB, len - t0);
+      if (t0) __syncthreads();
+      for (int i = threadIdx.x; i < tn * RMAX; i += 256) {
+        const int t = i / RMAX, r = i % RMAX;
+        a_s[i] = r < rank
+            ? hyb::to_f(proj[(row0 + t0 + t) * stride + a_off + r]) : 0.f;
+      }
+      __syncthreads();
+#pragma unroll 4
+      for (int t = 0; t < tn; ++t) {
+        float z = b;
+#pragma unroll
+        for (int r = 0; r < RMAX; ++r) z = fmaf(w[r], a_s[t * RMAX + r], z);
+        put_row(t0 + t, z);
+      }
+    }
+  } else {
+    for (int t = 0; t < len; ++t) {
+      const T *a = proj + (row0 + t) * stride + a_off;
+      float z = b;
+      for (int r = 0; r < rank; ++r)
+        z = fmaf(hyb::to_f(wr[r]), hyb::to_f(a[r]), z);
+      put_row(t, z);
+    }
   }
 }

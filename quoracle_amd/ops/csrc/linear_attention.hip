@@ -106,15 +106,15 @@ linear_recurrent_kernel(T *__restrict__ o, const T *__restrict__ proj,
         }
 #pragma unroll
         for (int i = 0; i < VEC; ++i) {
-          q[e * VEC + i] = hyb::activate(q[e * VEC + i], act);
-          k[e * VEC + i] = hyb::activate(k[e * VEC + i], act);
+          q[e * VEC + i] = hyb::activate<T>(q[e * VEC + i], act);
+          k[e * VEC + i] = hyb::activate<T>(k[e * VEC + i], act);
         }
       }
     }
 #pragma unroll
     for (int r = 0; r < RPT; ++r) {
       const int vi = v_base + r * RPG;
-      v[r] = vi < V ? hyb::activate(hyb::to_f(p[v_off + h * V + vi]), act)
+      v[r] = vi < V ? hyb::activate<T>(hyb::to_f(p[v_off + h * V + vi]), act)
                     : 0.f;
     }
 #pragma unroll
@@ -173,26 +173,40 @@ __device__ __forceinline__ bf16x8_t pack8(const float *v) {
   return __builtin_bit_cast(bf16x8_t, u);
 }
 
-// v = hi + lo + O(2^-17 v)
-__device__ __forceinline__ void split8(const float *v, bf16x8_t &hi,
-                                       bf16x8_t &lo) {
-  float r[8];
-#pragma unroll
-  for (int i = 0; i < 8; ++i) r[i] = v[i] - bf2f(f2bf(v[i]));
-  hi = pack8(v);
-  lo = pack8(r);
+// (a, b) = hi + lo + O(2^-17): two packed bf16 pairs
+__device__ __forceinline__ void split2(float a, float b, unsigned int &hi,
+                                       unsigned int &lo) {
+  hi = pack_bf16x2(a, b);
+  lo = pack_bf16x2(a - __uint_as_float(hi << 16),
+                   b - __uint_as_float(hi & 0xffff0000u));
 }
 
-// Eight activated elements, rounded to bf16 (the tiles' input precision).
+__device__ __forceinline__ void split8(const float *v, bf16x8_t &hi,
+                                       bf16x8_t &lo) {
+  uint4 h, l;
+  split2(v[0], v[1], h.x, l.x);
+  split2(v[2], v[3], h.y, l.y);
+  split2(v[4], v[5], h.z, l.z);
+  split2(v[6], v[7], h.w, l.w);
+  hi = __builtin_bit_cast(bf16x8_t, h);
+  lo = __builtin_bit_cast(bf16x8_t, l);
+}
+
+// Eight activated elements, to be rounded to bf16 by the caller.
 __device__ __forceinline__ void load8_act(const bf16 *p, bool ok, int act,
                                           float *o) {
   load8(p, ok, o);
   if (act != hyb::ACT_NONE) {
 #pragma unroll
-    for (int i = 0; i < 8; ++i)
-      o[i] = ok ? bf2f(f2bf(hyb::activate(o[i], act))) : 0.f;
+    for (int i = 0; i < 8; ++i) o[i] = hyb::activate<bf16>(o[i], act);
+    if (!ok) {          // the activation of zero need not be zero
+#pragma unroll
+      for (int i = 0; i < 8; ++i) o[i] = 0.f;
+    }
   }
 }
+
+__device__ __forceinline__ float round_bf16(float v) { return bf2f(f2bf(v)); }
 
 __device__ __forceinline__ f32x4_t mfma(const bf16x8_t &a, const bf16x8_t &b,
                                         const f32x4_t &c) {
@@ -206,9 +220,12 @@ __device__ __forceinline__ f32x4_t mfma(const bf16x8_t &a, const bf16x8_t &b,
 //   ws[chunk][h][v][d] = sum_j v_jv * (k_jd * decay from j to the end)
 //   decay: CH ? log decay summed along the chunk [rows, H*D]
 //             : powers of each head's decay [H][LIN_CHUNK + 1]
-// Grid: (chunks, H, ceil(D/64) * ceil(V/64)); block 256.
+// A workgroup forms TD key channels x TV value channels.  A thread stages two
+// neighbouring tokens at a time, so the [channel][token] images are written
+// in dwords.
+// Grid: (chunks, H, ceil(D/TD) * ceil(V/TV)); block 256.
 // ---------------------------------------------------------------------------
-template <bool CH>
+template <bool CH, int TD, int TV>
 __global__ void __launch_bounds__(256)
 linear_chunk_state_kernel(float *__restrict__ ws,
                           const bf16 *__restrict__ proj, long stride,
@@ -216,90 +233,104 @@ linear_chunk_state_kernel(float *__restrict__ ws,
                           const float *__restrict__ decay,
                           const int *__restrict__ chunk_row0,
                           const int *__restrict__ chunk_len) {
-  __shared__ __align__(16) bf16 v_s[64 * LIN_TS];
-  __shared__ __align__(16) bf16 k_hi[64 * LIN_TS];
-  __shared__ __align__(16) bf16 k_lo[64 * LIN_TS];
+  __shared__ __align__(16) bf16 v_s[TV * LIN_TS];
+  __shared__ __align__(16) bf16 k_hi[TD * LIN_TS];
+  __shared__ __align__(16) bf16 k_lo[TD * LIN_TS];
   const int chunk = blockIdx.x;
   const int h = blockIdx.y;
-  const int nd = (D + 63) / 64;
-  const int d0 = (blockIdx.z % nd) * 64;
-  const int v0 = (blockIdx.z / nd) * 64;
+  const int nd = (D + TD - 1) / TD;
+  const int d0 = (blockIdx.z % nd) * TD;
+  const int v0 = (blockIdx.z / nd) * TV;
   const long row0 = chunk_row0[chunk];
   const int L = chunk_len[chunk];
   const int tid = threadIdx.x;
-  const int j = tid & 63;
   const int wave = tid >> 6;
   const int lane = tid & 63;
-  const bool live = j < L;
+  const int j = (tid & 31) * 2;               // tokens j, j + 1
+  const int part = tid >> 5;                  // 8 channels of every 64
   const bf16 *p = proj + (row0 + j) * stride;
-  const float w_head = CH ? 0.f
-      : decay[h * (LIN_CHUNK + 1) + (live ? L - 1 - j : 0)];
+  const float *pw = decay + h * (LIN_CHUNK + 1);
 
 #pragma unroll
-  for (int half = 0; half < 2; ++half) {
-    const int c = wave * 16 + half * 8;
-    float kv[8], w[8];
-    const bool k_ok = live && d0 + c < D;
-    lin::load8_act(p + k_off + h * D + d0 + c, k_ok, act, kv);
-    if constexpr (CH) {
-      float end[8];
-      const long at = (row0 * H + h) * (long)D + d0 + c;
-      lin::load8f(decay + at + (long)(L - 1) * H * D, k_ok, end);
-      lin::load8f(decay + at + (long)j * H * D, k_ok, w);
+  for (int c = part * 8; c < TD; c += 64) {
+    float x[2][8];
 #pragma unroll
-      for (int e = 0; e < 8; ++e) w[e] = expf(end[e] - w[e]);
-    } else {
+    for (int u = 0; u < 2; ++u) {
+      const bool ok = j + u < L && d0 + c < D;
+      lin::load8_act(p + u * stride + k_off + h * D + d0 + c, ok, act, x[u]);
+      if constexpr (CH) {
+        float end[8], cj[8];
+        const long at = (row0 * H + h) * (long)D + d0 + c;
+        lin::load8f(decay + at + (long)(L - 1) * H * D, ok, end);
+        lin::load8f(decay + at + (long)(j + u) * H * D, ok, cj);
 #pragma unroll
-      for (int e = 0; e < 8; ++e) w[e] = w_head;
+        for (int e = 0; e < 8; ++e) x[u][e] *= __expf(end[e] - cj[e]);
+      } else {
+        const float w = ok ? pw[L - 1 - j - u] : 0.f;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) x[u][e] = lin::round_bf16(x[u][e]) * w;
+      }
     }
 #pragma unroll
     for (int e = 0; e < 8; ++e) {
-      const float x = kv[e] * w[e];
-      const bf16 hi = f2bf(x);
-      k_hi[(c + e) * LIN_TS + j] = hi;
-      k_lo[(c + e) * LIN_TS + j] = f2bf(x - bf2f(hi));
+      unsigned int hi, lo;
+      lin::split2(x[0][e], x[1][e], hi, lo);
+      *reinterpret_cast<unsigned int *>(k_hi + (c + e) * LIN_TS + j) = hi;
+      *reinterpret_cast<unsigned int *>(k_lo + (c + e) * LIN_TS + j) = lo;
     }
-    float vv[8];
-    lin::load8_act(p + v_off + h * V + v0 + c, live && v0 + c < V, act, vv);
+  }
 #pragma unroll
-    for (int e = 0; e < 8; ++e) v_s[(c + e) * LIN_TS + j] = f2bf(vv[e]);
+  for (int c = part * 8; c < TV; c += 64) {
+    float x[2][8];
+#pragma unroll
+    for (int u = 0; u < 2; ++u)
+      lin::load8_act(p + u * stride + v_off + h * V + v0 + c,
+                     j + u < L && v0 + c < V, act, x[u]);
+#pragma unroll
+    for (int e = 0; e < 8; ++e)
+      *reinterpret_cast<unsigned int *>(v_s + (c + e) * LIN_TS + j) =
+          pack_bf16x2(x[0][e], x[1][e]);
   }
   __syncthreads();
 
   const int fr = lane & 15, g = lane >> 4;
-  f32x4_t acc[4];
-#pragma unroll
-  for (int n = 0; n < 4; ++n) acc[n] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-  for (int kk = 0; kk < 2; ++kk) {
-    const int jo = kk * 32 + g * 8;
-    const bf16x8_t a = *reinterpret_cast<const bf16x8_t *>(
-        v_s + (wave * 16 + fr) * LIN_TS + jo);
-#pragma unroll
-    for (int n = 0; n < 4; ++n) {
-      acc[n] = lin::mfma(a, *reinterpret_cast<const bf16x8_t *>(
-          k_hi + (n * 16 + fr) * LIN_TS + jo), acc[n]);
-      acc[n] = lin::mfma(a, *reinterpret_cast<const bf16x8_t *>(
-          k_lo + (n * 16 + fr) * LIN_TS + jo), acc[n]);
-    }
-  }
   float *dst = ws + ((long)chunk * H + h) * (long)V * D;
 #pragma unroll
-  for (int r = 0; r < 4; ++r) {
-    const int v = v0 + wave * 16 + g * 4 + r;
-    if (v >= V) continue;
+  for (int vt = 0; vt < TV / 64; ++vt) {      // wave: 16 of every 64 values
+    const int vr = vt * 64 + wave * 16;
+    if (v0 + vr >= V) continue;               // wave-uniform
+    bf16x8_t a[2];
 #pragma unroll
-    for (int n = 0; n < 4; ++n) {
+    for (int kk = 0; kk < 2; ++kk)
+      a[kk] = *reinterpret_cast<const bf16x8_t *>(
+          v_s + (vr + fr) * LIN_TS + kk * 32 + g * 8);
+#pragma unroll
+    for (int n = 0; n < TD / 16; ++n) {
+      f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int kk = 0; kk < 2; ++kk) {
+        const int at = (n * 16 + fr) * LIN_TS + kk * 32 + g * 8;
+        acc = lin::mfma(a[kk], *reinterpret_cast<const bf16x8_t *>(k_hi + at),
+                        acc);
+        acc = lin::mfma(a[kk], *reinterpret_cast<const bf16x8_t *>(k_lo + at),
+                        acc);
+      }
       const int d = d0 + n * 16 + fr;
-      if (d < D) dst[(long)v * D + d] = acc[n][r];
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int v = v0 + vr + g * 4 + r;
+        if (v < V && d < D) dst[(long)v * D + d] = acc[r];
+      }
     }
   }
 }
 
 // ---------------------------------------------------------------------------
-// Scan along each sequence's chunks: ws[chunk] <- state at the chunk's start;
-// the state after the last chunk goes to the pool.  Four state elements per
-// thread, loads of four chunks in flight.
+// Scan along each sequence's chunks: ws[chunk] <- state at the chunk's start,
+// as the operand the output kernel reads (every four floats become four bf16
+// hi followed by their four bf16 lo, in place); the state after the last
+// chunk goes to the pool in float32.  Four state elements per thread, loads
+// of four chunks in flight.
 // Grid: (sequences, H, ceil(V*D / 1024)); block 256.
 // ---------------------------------------------------------------------------
 template <bool CH>
@@ -345,10 +376,14 @@ linear_chunk_scan_kernel(float *__restrict__ ws, float *__restrict__ state,
     for (int u = 0; u < 4; ++u) {
       const int c = cb + u;
       if (c < c1) {
-        hyb::store_v<4>(ws + ((long)c * H + h) * (long)VD + idx, S);
+        uint4 out;
+        lin::split2(S[0], S[1], out.x, out.z);
+        lin::split2(S[2], S[3], out.y, out.w);
+        *reinterpret_cast<uint4 *>(ws + ((long)c * H + h) * (long)VD + idx) =
+            out;
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-          const float f = CH ? expf(dec[u][i]) : dec[u][0];
+          const float f = CH ? __expf(dec[u][i]) : dec[u][0];
           S[i] = f * S[i] + own[u][i];
         }
       }
@@ -365,11 +400,12 @@ linear_chunk_scan_kernel(float *__restrict__ ws, float *__restrict__ state,
 // become the A operand of the value product in registers.
 //
 // CH scores: with c the log decay summed from the chunk's start, the factor
-// of channel d between i and j is exp(c_i - c_j).  Against the keys of an
-// earlier 16-row block it is split at the end of the block before the
-// wave's own rows, exp(c_i - c_ref) * exp(c_ref - c_j), both at most 1; in
-// the wave's own block it is formed pair by pair.  No factor can overflow,
-// whatever the decay.
+// of channel d between i and j is exp(c_i - c_j), split at the end of the
+// 16-row block before the wave's own rows: exp(c_i - c_ref), at most 1, times
+// exp(c_ref - c_j), at most 1 for keys of earlier blocks.  For keys of the
+// wave's own block the second factor is the inverse of the decay inside the
+// block; where that could leave the float range (a channel that loses more
+// than e^60 in 16 tokens) the block is formed pair by pair instead.
 // Grid: (chunks, H); block 256.  NK = ceil(D/32).
 // ---------------------------------------------------------------------------
 template <bool CH, int NK>
@@ -390,11 +426,12 @@ linear_chunk_out_kernel(bf16 *__restrict__ o, const float *__restrict__ ws,
   const int lane = tid & 63;
   const int fr = lane & 15, g = lane >> 4;
   const int qi = wave * 16 + fr;               // this lane's query row
+  const bool any = wave * 16 < L;              // this wave owns live rows
   const long HD = (long)H * D;
   const float *pw = decay + h * (LIN_CHUNK + 1);          // !CH
   const float *cum = decay + row0 * HD + (long)h * D;     // CH
 
-  // query operand(s): plain for !CH; decayed from the chunk's start for CH
+  // query operand: plain for !CH; decayed from the chunk's start for CH
   bf16x8_t q_hi[NK], q_lo[CH ? NK : 1];
   f32x4_t s[4];
 #pragma unroll
@@ -430,46 +467,68 @@ linear_chunk_out_kernel(bf16 *__restrict__ o, const float *__restrict__ ws,
   } else {
     const float *ci = cum + (long)min(qi, L - 1) * HD;
     const float *cref = cum + (long)(wave * 16 - 1) * HD;   // wave > 0
-    const bool any = wave * 16 < L;              // this wave owns live rows
+    const float *clast = cum + (long)min(wave * 16 + 15, L - 1) * HD;
+    float drop = 0.f;                // most any channel loses in own block
 #pragma unroll
     for (int kk = 0; kk < NK; ++kk) {
       const int d = kk * 32 + g * 8;
-      const bool ok = any && qi < L && d < D;
+      float ref[8], last[8];
+      lin::load8f(cref + d, wave > 0 && any && d < D, ref);
+      lin::load8f(clast + d, d < D, last);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) drop = fmaxf(drop, ref[e] - last[e]);
+    }
+    const bool tame = !__any(any && drop > 60.f);           // wave-uniform
+#pragma unroll
+    for (int kk = 0; kk < NK; ++kk) {
+      const int d = kk * 32 + g * 8;
+      const bool ok = qi < L && d < D;
       float q[8], c[8], x[8], ref[8];
+      bf16x8_t a_hi, a_lo;
       lin::load8_act(qp + d, ok, act, q);
       lin::load8f(ci + d, ok, c);
+      lin::load8f(cref + d, wave > 0 && any && d < D, ref);
 #pragma unroll
-      for (int e = 0; e < 8; ++e) x[e] = q[e] * expf(c[e]);
-      lin::split8(x, q_hi[kk], q_lo[kk]);
-      if (any && wave > 0) {                     // wave-uniform
-        bf16x8_t a_hi, a_lo;
-        lin::load8f(cref + d, d < D, ref);
+      for (int e = 0; e < 8; ++e) x[e] = q[e] * __expf(c[e] - ref[e]);
+      if (!ok) {
 #pragma unroll
-        for (int e = 0; e < 8; ++e) x[e] = ok ? q[e] * expf(c[e] - ref[e])
-                                              : 0.f;
-        lin::split8(x, a_hi, a_lo);
+        for (int e = 0; e < 8; ++e) x[e] = 0.f;
+      }
+      lin::split8(x, a_hi, a_lo);
+      if (wave == 0) {                           // the start is the reference
+        q_hi[kk] = a_hi;
+        q_lo[kk] = a_lo;
+      } else {
 #pragma unroll
-        for (int J = 0; J < 3; ++J) {
-          if (J >= wave) continue;
-          const int j = J * 16 + fr;             // < wave*16 <= L
-          float k[8], cj[8];
-          bf16x8_t b_hi, b_lo;
-          lin::load8_act(proj + (row0 + j) * stride + k_off + h * D + d,
-                         d < D, act, k);
-          lin::load8f(cum + (long)j * HD + d, d < D, cj);
+        for (int e = 0; e < 8; ++e) x[e] = q[e] * __expf(c[e]);
+        lin::split8(x, q_hi[kk], q_lo[kk]);
+      }
 #pragma unroll
-          for (int e = 0; e < 8; ++e) k[e] *= expf(ref[e] - cj[e]);
-          lin::split8(k, b_hi, b_lo);
-          s[J] = lin::mfma(b_hi, a_hi, s[J]);
-          s[J] = lin::mfma(b_lo, a_hi, s[J]);
-          s[J] = lin::mfma(b_hi, a_lo, s[J]);
+      for (int J = 0; J < 4; ++J) {
+        if (J > wave || J * 16 >= L || (J == wave && !tame)) continue;
+        const int j = J * 16 + fr;
+        const bool k_ok = j < L && d < D;
+        float k[8], cj[8];
+        bf16x8_t b_hi, b_lo;
+        lin::load8_act(proj + (row0 + min(j, L - 1)) * stride + k_off + h * D
+                           + d, k_ok, act, k);
+        lin::load8f(cum + (long)min(j, L - 1) * HD + d, k_ok, cj);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) k[e] *= __expf(ref[e] - cj[e]);
+        if (!k_ok) {
+#pragma unroll
+          for (int e = 0; e < 8; ++e) k[e] = 0.f;
         }
+        lin::split8(k, b_hi, b_lo);
+        s[J] = lin::mfma(b_hi, a_hi, s[J]);
+        s[J] = lin::mfma(b_lo, a_hi, s[J]);
+        s[J] = lin::mfma(b_hi, a_lo, s[J]);
       }
     }
-    // own block, pair by pair in float32: this lane's query against keys
-    // wave*16 + g*4 + r
-    if (any) {
-      float dot[4] = {0.f, 0.f, 0.f, 0.f};
+    float dot[4] = {0.f, 0.f, 0.f, 0.f};
+    if (!tame) {
+      // own block, pair by pair: this lane's query against keys
+      // wave*16 + g*4 + r
       for (int d = 0; d < D; d += 8) {
         float q[8], c[8];
         lin::load8_act(qp + d, true, act, q);
@@ -487,14 +546,15 @@ linear_chunk_out_kernel(bf16 *__restrict__ o, const float *__restrict__ ws,
                           dot[r]);
         }
       }
+    }
 #pragma unroll
-      for (int J = 0; J < 4; ++J) {
-        if (J != wave) continue;
+    for (int J = 0; J < 4; ++J) {
+      if (J != wave) continue;
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int key = J * 16 + g * 4 + r;
-          s[J][r] = (key <= qi && qi < L) ? dot[r] : 0.f;
-        }
+      for (int r = 0; r < 4; ++r) {
+        const int key = J * 16 + g * 4 + r;
+        const float v = tame ? s[J][r] : dot[r];
+        s[J][r] = (key <= qi && qi < L) ? v : 0.f;
       }
     }
   }
@@ -511,30 +571,39 @@ linear_chunk_out_kernel(bf16 *__restrict__ o, const float *__restrict__ ws,
   for (int v0 = 0; v0 < V; v0 += 64) {
     if (v0) __syncthreads();
     {
-      const int j = tid & 63;
-      const bf16 *vp = proj + (row0 + min(j, L - 1)) * stride + v_off + h * V;
+      const int j = (tid & 31) * 2;            // tokens j, j + 1
+      const int c = (tid >> 5) * 8;
+      float x[2][8];
 #pragma unroll
-      for (int half = 0; half < 2; ++half) {
-        const int c = wave * 16 + half * 8;
-        float vv[8];
-        lin::load8_act(vp + v0 + c, j < L && v0 + c < V, act, vv);
+      for (int u = 0; u < 2; ++u)
+        lin::load8_act(proj + (row0 + min(j + u, L - 1)) * stride + v_off
+                           + h * V + v0 + c, j + u < L && v0 + c < V, act,
+                       x[u]);
 #pragma unroll
-        for (int e = 0; e < 8; ++e) v_s[(c + e) * LIN_TS + j] = f2bf(vv[e]);
-      }
+      for (int e = 0; e < 8; ++e)
+        *reinterpret_cast<unsigned int *>(v_s + (c + e) * LIN_TS + j) =
+            pack_bf16x2(x[0][e], x[1][e]);
     }
     __syncthreads();
 #pragma unroll
     for (int vt = 0; vt < 4; ++vt) {
       const int vb = v0 + vt * 16;
-      if (vb >= V || wave * 16 >= L) continue;   // wave-uniform
+      if (vb >= V || !any) continue;           // wave-uniform
       f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int kk = 0; kk < NK; ++kk) {
         const int d = kk * 32 + g * 8;
-        float x[8];
-        bf16x8_t s_hi, s_lo;
-        lin::load8f(S + (long)(vb + fr) * D + d, vb + fr < V && d < D, x);
-        lin::split8(x, s_hi, s_lo);
+        uint4 x = make_uint4(0, 0, 0, 0), y = x;
+        if (vb + fr < V && d < D) {
+          const uint4 *at = reinterpret_cast<const uint4 *>(
+              S + (long)(vb + fr) * D + d);
+          x = at[0];
+          y = at[1];
+        }
+        const bf16x8_t s_hi = __builtin_bit_cast(
+            bf16x8_t, make_uint4(x.x, x.y, y.x, y.y));
+        const bf16x8_t s_lo = __builtin_bit_cast(
+            bf16x8_t, make_uint4(x.z, x.w, y.z, y.w));
         acc = lin::mfma(q_hi[kk], s_hi, acc);
         acc = lin::mfma(q_hi[kk], s_lo, acc);
         if constexpr (CH) acc = lin::mfma(q_lo[kk], s_hi, acc);

@@ -211,12 +211,20 @@ void qk_norm_rope_store(Tensor q_out, Tensor kcache, Tensor vcache,
   if (T == 0) return;
   by_dtype(q_out, [&](auto t0) {
     using A = decltype(t0);
-    qk_norm_rope_store_kernel<A>
-        <<<dim3(T), dim3(256), 2 * pairs * sizeof(float), current_stream()>>>(
-            ptr<A>(q_out), ptr<A>(kcache), ptr<A>(vcache), ptr<A>(proj),
-            stride, (int)q_off, (int)k_off, fptr(qw), fptr(kw),
-            iptr(positions), iptr(slots), freq.data_ptr<double>(), pairs, (float)mag,
-            (float)eps, H, G, D, BS);
+    auto run = [&](auto kernel) {
+      kernel<<<dim3(T), dim3(256), 2 * pairs * sizeof(float),
+               current_stream()>>>(
+          ptr<A>(q_out), ptr<A>(kcache), ptr<A>(vcache), ptr<A>(proj), stride,
+          (int)q_off, (int)k_off, fptr(qw), fptr(kw), iptr(positions),
+          iptr(slots), freq.data_ptr<double>(), pairs, (float)mag, (float)eps,
+          H, G, D, BS);
+    };
+    const long groups = (long)(H + G) * D / 8;
+    if (D % 8 || stride % 8 || q_off % 8 || k_off % 8 || groups > 4 * 256)
+      run(qk_norm_rope_store_kernel<A>);
+    else if (groups <= 256) run(qk_norm_rope_store8_kernel<A, 1>);
+    else if (groups <= 512) run(qk_norm_rope_store8_kernel<A, 2>);
+    else run(qk_norm_rope_store8_kernel<A, 4>);
   });
   HIP_CHECK_KERNEL();
 }
@@ -242,7 +250,7 @@ void log_decay(Tensor out, Tensor proj, int64_t a_off, Tensor a2, Tensor bias,
     using A = decltype(t0);
     auto run = [&](auto rmax) {
       log_decay_kernel<A, decltype(rmax)::value>
-          <<<dim3(runs, (C + 255) / 256), dim3(256), 0, current_stream()>>>(
+          <<<dim3(runs, (C + 63) / 64), dim3(256), 0, current_stream()>>>(
               fptr(out) + first * C, ptr<A>(proj) + first * stride, stride,
               (int)a_off, rank, ptr<A>(a2), fptr(bias), (float)(1.0 / tau),
               C, run_row0 ? iptr(*run_row0) : nullptr,
@@ -498,13 +506,8 @@ void linear_chunked(Tensor o, Tensor proj, int64_t q_off, int64_t k_off,
               a.D, a.V, (int)act, fptr(decay), iptr(chunk_row0),
               iptr(chunk_len));
     };
-    if (a.D <= 64) {
-      if (a.V <= 64) state(Int<64>(), Int<64>());
-      else state(Int<64>(), Int<128>());
-    } else {
-      if (a.V <= 64) state(Int<128>(), Int<64>());
-      else state(Int<128>(), Int<128>());
-    }
+    if (a.V <= 64) state(Int<64>(), Int<64>());
+    else state(Int<64>(), Int<128>());
     HIP_CHECK_KERNEL();
     linear_chunk_scan_kernel<CH><<<g_scan, dim3(256), 0, stream>>>(
         fptr(ws), fptr(state_pool), a.H, a.D, a.V, fptr(decay), iptr(chunk_row0),

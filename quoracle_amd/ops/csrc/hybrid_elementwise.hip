@@ -321,15 +321,118 @@ qk_norm_rope_store_kernel(
   }
 }
 
+// The same for head dimensions, offsets and rows that are multiples of 8:
+// eight elements (four pairs) at a time, the token's groups held in
+// registers.  NI groups per thread.
+template <typename T, int NI>
+__global__ void __launch_bounds__(256)
+qk_norm_rope_store8_kernel(
+    T *__restrict__ q_out, T *__restrict__ kcache, T *__restrict__ vcache,
+    const T *__restrict__ proj, long stride, int q_off, int k_off,
+    const float *__restrict__ qw, const float *__restrict__ kw,
+    const int *__restrict__ positions, const int *__restrict__ slots,
+    const double *__restrict__ freq, int n_pairs, float mag, float eps, int H,
+    int G, int D, int BS) {
+  extern __shared__ float rot_s[];
+  __shared__ float scratch[8];
+  float *cos_s = rot_s, *sin_s = rot_s + n_pairs;
+  const long t = blockIdx.x;
+  const int tid = threadIdx.x;
+  const T *row = proj + t * stride;
+  const int nq = H * D, nk = G * D, n8 = (nq + nk) / 8;
+  float x[NI][8];
+  float sq = 0.f, sk = 0.f;
+#pragma unroll
+  for (int it = 0; it < NI; ++it) {
+    const int i = (it * 256 + tid) * 8;
+    if (i >= n8 * 8) continue;
+    hyb::load_v<8>(row + (i < nq ? q_off + i : k_off + i - nq), x[it]);
+    float s = 0.f;
+#pragma unroll
+    for (int k = 0; k < 8; ++k) s += x[it][k] * x[it][k];
+    if (i < nq) sq += s;
+    else sk += s;
+  }
+  const double pos = (double)positions[t];
+  for (int i = tid; i < n_pairs; i += 256) {
+    double turns = pos * freq[i] * 0.15915494309189535;
+    turns -= rint(turns);
+    float s, c;
+    sincosf((float)(turns * 6.283185307179586), &s, &c);
+    cos_s[i] = c * mag;
+    sin_s[i] = s * mag;
+  }
+  sq = wave_sum(sq);
+  sk = wave_sum(sk);
+  if ((tid & 63) == 0) {
+    scratch[tid >> 6] = sq;
+    scratch[4 + (tid >> 6)] = sk;
+  }
+  __syncthreads();                     // also publishes cos_s / sin_s
+  sq = scratch[0] + scratch[1] + scratch[2] + scratch[3];
+  sk = scratch[4] + scratch[5] + scratch[6] + scratch[7];
+  const float qi = 1.f / sqrtf(sq / (float)nq + eps);
+  const float ki = 1.f / sqrtf(sk / (float)nk + eps);
+  const int slot = slots[t];
+  const long blk = slot / BS;
+  const int off = slot % BS;
+#pragma unroll
+  for (int it = 0; it < NI; ++it) {
+    const int i = (it * 256 + tid) * 8;
+    if (i >= n8 * 8) continue;
+    const bool is_q = i < nq;
+    const int at = is_q ? i : i - nq;
+    const int head = at / D, d = at % D;
+    const float inv = is_q ? qi : ki;
+    float w[8], y[8];
+    hyb::load_v<8>((is_q ? qw : kw) + at, w);
+#pragma unroll
+    for (int k = 0; k < 8; ++k) y[k] = x[it][k] * inv * w[k];
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      const int pr = d / 2 + k;
+      if (pr < n_pairs) {
+        const float c = cos_s[pr], s = sin_s[pr];
+        const float u = y[2 * k], v = y[2 * k + 1];
+        y[2 * k] = u * c - v * s;
+        y[2 * k + 1] = v * c + u * s;
+      }
+    }
+    if (is_q) {
+      hyb::store_v<8>(q_out + t * nq + at, y);
+    } else if (slot >= 0) {
+      const long dst = ((blk * G + head) * (long)BS + off) * D + d;
+      hyb::store_v<8>(kcache + dst, y);
+      hyb::store_v<8>(vcache + dst, x[it]);
+    }
+  }
+}
+
 // ---------------------------------------------------------------------------
 // Log of a low-rank sigmoid decay per key channel, summed along runs of
 // consecutive rows:
 //   z = A2 a1[t] + b,  ld[t] = log(sigmoid(z)) / tau,
 //   out[t] = ld[t] + out[t-1] inside a run (the first row of a run: ld[t]).
 // run_row0 null: every row is a run of its own (out = ld).
-// Grid: (runs, ceil(C/256)); block 256, one channel per thread.
+// A workgroup takes 64 channels; its four waves take 16 rows each of every 64
+// and join their sums.  RMAX: rank the channel's weights are held in
+// registers for; 0: any rank.
+// Grid: (runs, ceil(C/64)); block 256.
 // ---------------------------------------------------------------------------
-// RMAX: rank the channel's weights are held in registers for; 0: any rank.
+// log(sigmoid(z)) = min(z, 0) - log(1 + e), e = exp(-|z|).  For bf16 models
+// with the hardware exponential and logarithm, and the series of log(1 + e)
+// where 1 + e would round away e (both within 2^-20 of the value).
+template <typename T> __device__ __forceinline__ float log_sigmoid(float z) {
+  if constexpr (sizeof(T) == 2) {
+    const float e = __expf(-fabsf(z));
+    const float series =
+        e * (1.f - e * (0.5f - e * (0.33333333f - e * (0.25f - e * 0.2f))));
+    return fminf(z, 0.f) - (e < 0.0625f ? series : __logf(1.f + e));
+  } else {
+    return fminf(z, 0.f) - log1pf(expf(-fabsf(z)));
+  }
+}
+
 template <typename T, int RMAX>
 __global__ void __launch_bounds__(256)
 log_decay_kernel(float *__restrict__ out, const T *__restrict__ proj,
@@ -337,49 +440,69 @@ log_decay_kernel(float *__restrict__ out, const T *__restrict__ proj,
                  const float *__restrict__ bias, float inv_tau, int C,
                  const int *__restrict__ run_row0,
                  const int *__restrict__ run_len) {
-  constexpr int TB = 64;                       // rows staged at a time
+  constexpr int TB = 64;
   constexpr int RS = RMAX ? RMAX : 1;
   __shared__ __align__(16) float a_s[TB * RS];
-  const int c = min((int)(blockIdx.y * 256 + threadIdx.x), C - 1);
-  const bool live = blockIdx.y * 256 + threadIdx.x < C;
+  __shared__ float sum_s[4][64];
+  const int lane = threadIdx.x & 63;
+  const int quarter = threadIdx.x >> 6;
+  const int c = min((int)blockIdx.y * 64 + lane, C - 1);
+  const bool live = (int)blockIdx.y * 64 + lane < C;
   const long row0 = run_row0 ? run_row0[blockIdx.x] : (int)blockIdx.x;
   const int len = run_row0 ? run_len[blockIdx.x] : 1;
   const T *wr = a2 + (long)c * rank;
   const float b = bias[c];
   float w[RS];
+  if (RMAX > 0 && quarter * 16 < len) {
+    if (rank == RMAX) {
 #pragma unroll
-  for (int r = 0; r < RS; ++r) w[r] = r < rank ? hyb::to_f(wr[r]) : 0.f;
-  float sum = 0.f;
-  auto put_row = [&](int t, float z) {
-    const float ls = fminf(z, 0.f) - log1pf(expf(-fabsf(z)));
-    sum += ls * inv_tau;
-    if (live) out[(row0 + t) * (long)C + c] = sum;
-  };
-  if constexpr (RMAX > 0) {
-    for (int t0 = 0; t0 < len; t0 += TB) {
-      const int tn = min(TB, len - t0);
-      if (t0) __syncthreads();
+      for (int r = 0; r < RS / 8; ++r) hyb::load_v<8>(wr + 8 * r, w + 8 * r);
+    } else {
+#pragma unroll
+      for (int r = 0; r < RS; ++r) w[r] = r < rank ? hyb::to_f(wr[r]) : 0.f;
+    }
+  }
+  float carry = 0.f;
+  for (int t0 = 0; t0 < len; t0 += TB) {
+    const int tn = min(TB, len - t0);
+    const T *a = proj + (row0 + t0) * stride + a_off;
+    if constexpr (RMAX > 0) {
       for (int i = threadIdx.x; i < tn * RMAX; i += 256) {
         const int t = i / RMAX, r = i % RMAX;
-        a_s[i] = r < rank
-            ? hyb::to_f(proj[(row0 + t0 + t) * stride + a_off + r]) : 0.f;
+        a_s[i] = r < rank ? hyb::to_f(a[t * stride + r]) : 0.f;
       }
       __syncthreads();
-#pragma unroll 4
-      for (int t = 0; t < tn; ++t) {
-        float z = b;
+    }
+    float part[16], sum = 0.f;
 #pragma unroll
-        for (int r = 0; r < RMAX; ++r) z = fmaf(w[r], a_s[t * RMAX + r], z);
-        put_row(t0 + t, z);
+    for (int u = 0; u < 16; ++u) {
+      const int t = quarter * 16 + u;
+      if (t < tn) {                                   // wave-uniform
+        float z = b;
+        if constexpr (RMAX > 0) {
+#pragma unroll
+          for (int r = 0; r < RMAX; ++r) z = fmaf(w[r], a_s[t * RMAX + r], z);
+        } else {
+          for (int r = 0; r < rank; ++r)
+            z = fmaf(hyb::to_f(wr[r]), hyb::to_f(a[t * stride + r]), z);
+        }
+        sum += log_sigmoid<T>(z) * inv_tau;
       }
+      part[u] = sum;
     }
-  } else {
-    for (int t = 0; t < len; ++t) {
-      const T *a = proj + (row0 + t) * stride + a_off;
-      float z = b;
-      for (int r = 0; r < rank; ++r)
-        z = fmaf(hyb::to_f(wr[r]), hyb::to_f(a[r]), z);
-      put_row(t, z);
+    sum_s[quarter][lane] = sum;
+    __syncthreads();
+    float before = carry;
+#pragma unroll
+    for (int q = 0; q < 4; ++q) {
+      if (q < quarter) before += sum_s[q][lane];
+      carry += sum_s[q][lane];
     }
+#pragma unroll
+    for (int u = 0; u < 16; ++u) {
+      const int t = quarter * 16 + u;
+      if (t < tn && live) out[(row0 + t0 + t) * (long)C + c] = before + part[u];
+    }
+    if (t0 + TB < len) __syncthreads();
   }
 }

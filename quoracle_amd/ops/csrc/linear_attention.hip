@@ -409,7 +409,7 @@ linear_chunk_scan_kernel(float *__restrict__ ws, float *__restrict__ state,
 // Grid: (chunks, H); block 256.  NK = ceil(D/32).
 // ---------------------------------------------------------------------------
 template <bool CH, int NK>
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(256, CH ? (NK > 4 ? 2 : 3) : 4)
 linear_chunk_out_kernel(bf16 *__restrict__ o, const float *__restrict__ ws,
                         const bf16 *__restrict__ proj, long stride, int q_off,
                         int k_off, int v_off, int H, int D, int V, int act,

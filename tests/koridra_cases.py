@@ -71,6 +71,14 @@ CONFIGS = {
                  "right": {"heads": 2, "dim": 32, "vdim": 96, "tau": 2.0},
                  "left_scale": 0.5, "right_scale": 0.8}},
         ]},
+    # no attention at all: no pages' bytes, only states
+    "recurrent": {
+        "architecture": "Koridra", "vocab": 280, "width": 40,
+        "max_positions": 400, "postln_alpha": 1.2, "norm": {"eps": 1e-4},
+        "layers": [
+            {"type": "lightning", "mlp": {"kind": "dense", "ff": 56},
+             "mixer": {"heads": 1, "dim": 48, "vdim": 136,
+                       "decay": [0.98]}}]},
 }
 RANKS = {"tiles": 4, "odd": 3, "wide": 21}
 

@@ -161,9 +161,8 @@ gated_norm_kernel(T *__restrict__ out, const T *__restrict__ o,
   const long t = blockIdx.x;
   const long base = (t * gridDim.y + blockIdx.y) * (long)n;
   const T *gate = proj + t * stride + g_off + (long)blockIdx.y * n;
-  auto finish = [&](int i, float *v, float inv) {
-    float gv[VEC], wv[VEC];
-    hyb::load_v<VEC>(gate + i, gv);
+  auto finish = [&](int i, float *v, const float *gv, float inv) {
+    float wv[VEC];
     hyb::load_v<VEC>(w + i, wv);
 #pragma unroll
     for (int k = 0; k < VEC; ++k)
@@ -172,12 +171,13 @@ gated_norm_kernel(T *__restrict__ out, const T *__restrict__ o,
   };
   float ssq = 0.f;
   if constexpr (NI > 0) {
-    float v[NI][VEC];
+    float v[NI][VEC], gv[NI][VEC];       // the gate is on its way meanwhile
 #pragma unroll
     for (int it = 0; it < NI; ++it) {
       const int i = (it * 256 + threadIdx.x) * VEC;
       if (i >= n) continue;
       hyb::load_v<VEC>(o + base + i, v[it]);
+      hyb::load_v<VEC>(gate + i, gv[it]);
 #pragma unroll
       for (int k = 0; k < VEC; ++k) ssq += v[it][k] * v[it][k];
     }
@@ -185,7 +185,7 @@ gated_norm_kernel(T *__restrict__ out, const T *__restrict__ o,
 #pragma unroll
     for (int it = 0; it < NI; ++it) {
       const int i = (it * 256 + threadIdx.x) * VEC;
-      if (i < n) finish(i, v[it], inv);
+      if (i < n) finish(i, v[it], gv[it], inv);
     }
   } else {
     for (int i = threadIdx.x * VEC; i < n; i += 256 * VEC) {
@@ -196,9 +196,10 @@ gated_norm_kernel(T *__restrict__ out, const T *__restrict__ o,
     }
     const float inv = 1.f / sqrtf(block_sum(ssq, scratch) / (float)n + eps);
     for (int i = threadIdx.x * VEC; i < n; i += 256 * VEC) {
-      float v[VEC];
+      float v[VEC], gv[VEC];
       hyb::load_v<VEC>(o + base + i, v);
-      finish(i, v, inv);
+      hyb::load_v<VEC>(gate + i, gv);
+      finish(i, v, gv, inv);
     }
   }
 }
@@ -214,10 +215,13 @@ gated_norm_small_kernel(T *__restrict__ out, const T *__restrict__ o,
   const long at = ((long)blockIdx.x * 256 + threadIdx.x) / LPG;
   const int i = (threadIdx.x % LPG) * VEC;
   const bool live = at < total && i < n;
-  float v[VEC];
+  float v[VEC], gv[VEC], wv[VEC];
   float ssq = 0.f;
   if (live) {
     hyb::load_v<VEC>(o + at * n + i, v);
+    hyb::load_v<VEC>(
+        proj + at / groups * stride + g_off + at % groups * n + i, gv);
+    hyb::load_v<VEC>(w + i, wv);
 #pragma unroll
     for (int k = 0; k < VEC; ++k) ssq += v[k] * v[k];
   }
@@ -225,10 +229,6 @@ gated_norm_small_kernel(T *__restrict__ out, const T *__restrict__ o,
   for (int s = LPG / 2; s >= 1; s >>= 1) ssq += __shfl_xor(ssq, s, LPG);
   if (!live) return;
   const float inv = 1.f / sqrtf(ssq / (float)n + eps);
-  float gv[VEC], wv[VEC];
-  hyb::load_v<VEC>(proj + at / groups * stride + g_off + at % groups * n + i,
-                   gv);
-  hyb::load_v<VEC>(w + i, wv);
 #pragma unroll
   for (int k = 0; k < VEC; ++k)
     v[k] = v[k] * inv * wv[k] * hyb::activate<T>(gv[k], act);

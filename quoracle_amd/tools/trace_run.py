@@ -4,8 +4,8 @@
 
 Steps come from standard input, one JSON object a line:
 
-  {"step": 0, "entries": [{"id": "a", "tokens": [5, 17, 3], "want": [0, 2]}],
-   "end": []}
+  {"step": 4, "entries": [{"id": "x", "tokens": [40, 7], "want": [1]}],
+   "end": ["y"]}
 
 All entries of a step are one batch of the engine (LocalEngine.step_entries:
 the step, cache, state slots and kernels of generation; decode-only steps
@@ -88,7 +88,7 @@ def main(argv: Optional[List[str]] = None) -> int:
                    default="bfloat16")
     p.add_argument("--out", required=True, help="folder for <step>.f32")
     p.add_argument("--max-tokens", type=int, required=True,
-                   help="most tokens that live requests hold at any time")
+                   help="size of the K/V pool in tokens")
     p.add_argument("--device", default=None,
                    help="cpu: the plain implementations, for tests")
     a = p.parse_args(argv)

@@ -531,8 +531,11 @@ class LocalEngine(Engine):
         starts: List[int] = []
         slots: List[int] = []
         placed: List[BatchEntry] = []
-        for e in ([e for e in entries if len(e.tokens) == 1]
-                  + [e for e in entries if len(e.tokens) > 1]):
+        # single tokens first, then portions; where the model treats short
+        # portions differently, those before the long ones
+        split = getattr(hm.model, "expand_from", None) or 2
+        for e in sorted(entries, key=lambda e: (len(e.tokens) > 1)
+                        + (len(e.tokens) >= split)):
             start = len(e.session.token_ids)
             try:
                 slots.extend(hm.sessions.extend(e.session, e.tokens,
@@ -606,6 +609,12 @@ class LocalEngine(Engine):
         seg: Dict[str, List[int]] = {"row0": [], "len": [], "chunk0": [0]}
         chunk: Dict[str, List[int]] = {"row0": [], "len": []}
         max_kv = 0
+        # portions this long attend over keys and values made from the cached
+        # latents of their whole context; shorter ones take 16-row tiles
+        split = getattr(hm.model, "expand_from", None)
+        ctx_slots: List[np.ndarray] = []
+        ctx0: List[int] = []
+        n_ctx, n_latent = 0, n_decode
         for i, (e, start) in enumerate(zip(placed, starts)):
             row, n = len(tokens), len(e.tokens)
             tokens.extend(e.tokens)
@@ -617,14 +626,26 @@ class LocalEngine(Engine):
             if i < n_decode:
                 continue
             max_kv = max(max_kv, start + n)
-            for name, step in (("tile", QT), ("tile32", big_step)):
-                if name == "tile" and hm.cfg.is_hybrid:
-                    continue
+            if not hm.cfg.is_hybrid:
+                kinds = (("tile", QT), ("tile32", big_step))
+            elif split is not None and n < split:
+                kinds = (("tile", QT),)
+                n_latent = row + n
+            else:
+                kinds = (("tile32", big_step),)
+            for name, step in kinds:
                 for off in range(0, n, step):
                     tiles[name + "_q0"].append(row + off)
                     tiles[name + "_qn"].append(min(step, n - off))
                     tiles[name + "_seq"].append(i)
                     tiles[name + "_pos0"].append(start + off)
+            if split is not None and n >= split:
+                at = np.arange(start + n)
+                blocks = np.asarray(e.session.blocks, dtype=np.int32)
+                ctx_slots.append(blocks[at // BLOCK_SIZE] * BLOCK_SIZE
+                                 + at % BLOCK_SIZE)
+                ctx0 += [n_ctx] * -(-n // big_step)
+                n_ctx += start + n
             seg["row0"].append(row)
             seg["len"].append(n)
             for off in range(0, n, LIN_CHUNK):
@@ -643,11 +664,16 @@ class LocalEngine(Engine):
         if n_decode:
             arrays["ctx_lens"] = [s + 1 for s in starts[:n_decode]]
         if hm.cfg.is_hybrid:
+            arrays["row_seq"] = row_seq
+        if hm.cfg.needs_state:
             arrays.update(
-                row_seq=row_seq, seg_row0=seg["row0"], seg_len=seg["len"],
+                seg_row0=seg["row0"], seg_len=seg["len"],
                 seg_chunk0=seg["chunk0"], chunk_row0=chunk["row0"],
                 chunk_len=chunk["len"],
                 state_slots=[e.session.state_slot for e in placed])
+        if ctx_slots:
+            arrays["ctx_slots"] = np.concatenate(ctx_slots)
+            arrays["tile32_ctx0"] = ctx0
 
         t_fwd = time.monotonic()
         # rocprof/omnitrace attribution: roctx ranges around each eager
@@ -660,7 +686,8 @@ class LocalEngine(Engine):
         with hm.stream_ctx():
             batch = ForwardBatch(
                 n_decode=n_decode, max_ctx=max(starts[:n_decode], default=-1)
-                + 1, max_kv=max_kv, **_to_device(arrays, dev))
+                + 1, max_kv=max_kv, n_latent=n_latent,
+                **_to_device(arrays, dev))
             hidden = hm.model.forward(batch, hm.kv)
             logits = None
             if sample_rows:

@@ -79,7 +79,7 @@ class DecodeGraphs:
             batch = ForwardBatch(
                 tokens=bufs["tokens"], positions=bufs["positions"],
                 slots=bufs["slots"], block_tables=bufs["block_tables"],
-                n_decode=bucket, ctx_lens=bufs["ctx_lens"],
+                n_decode=bucket, n_latent=bucket, ctx_lens=bufs["ctx_lens"],
                 max_ctx=1 << 30,     # force the split decode path (NS fixed)
                 row_seq=row_seq, state_slots=bufs.get("state_slots"))
             hidden = self.model.forward(batch, self.kv)

@@ -18,7 +18,8 @@ import os
 from dataclasses import dataclass
 from typing import Dict, Union
 
-from .hybrid_config import KoridraConfig, koridra_preset
+from .hybrid_config import (HybridConfig, KoridraConfig, KotutarConfig,
+                            LoopSpec, koridra_preset, kotutar_preset)
 
 
 @dataclass(frozen=True)
@@ -78,7 +79,7 @@ class ModelConfig:
         return embed + lm_head + self.n_layers * per_layer + self.hidden
 
 
-AnyConfig = Union[ModelConfig, KoridraConfig]
+AnyConfig = Union[ModelConfig, HybridConfig]
 
 PRESETS: Dict[str, AnyConfig] = {
     # CPU-testable toy model (head_dim multiple of 8, <=128 for the kernels)
@@ -139,10 +140,28 @@ PRESETS: Dict[str, AnyConfig] = {
         "koridra-8b", vocab=128256, hidden=4096, n_layers=32, ff=14336,
         heads=32, kv_heads=8, dim=128, chunk=8192, lin_heads=32, lin_dim=128,
         lin_vdim=128, max_context=32768),
+    # CPU-testable Kotutar toy
+    "kotutar-tiny": kotutar_preset(
+        "kotutar-tiny", vocab=512, hidden=64, n_layers=4, ff=96, heads=3,
+        dim=16, rot_dim=8, vdim=24, q_rank=40, kv_rank=32, experts=5, top=2,
+        expert_ff=48, shared_ff=56, loop=LoopSpec(1, 3, 2),
+        max_context=4096, max_output=1024, base=10000.0),
+    # Kotutar with the layer sizes of a 1B-class and of an 8B-class model
+    "kotutar-1b": kotutar_preset(
+        "kotutar-1b", vocab=128256, hidden=2048, n_layers=16, ff=8192,
+        heads=16, dim=128, rot_dim=64, vdim=128, q_rank=768, kv_rank=512,
+        experts=16, top=2, expert_ff=2048, shared_ff=2048,
+        loop=LoopSpec(4, 12, 2)),
+    "kotutar-8b": kotutar_preset(
+        "kotutar-8b", vocab=128256, hidden=4096, n_layers=32, ff=14336,
+        heads=32, dim=128, rot_dim=64, vdim=128, q_rank=1536, kv_rank=512,
+        experts=16, top=2, expert_ff=4096, shared_ff=4096,
+        loop=LoopSpec(8, 24, 2)),
 }
 
 # config.json "architecture" -> reader of the rest of the file
-ARCHITECTURES = {"Koridra": KoridraConfig.from_dict}
+ARCHITECTURES = {"Koridra": KoridraConfig.from_dict,
+                 "Kotutar": KotutarConfig.from_dict}
 
 
 @functools.lru_cache(maxsize=64)

@@ -68,6 +68,11 @@ class ForwardBatch:
     seg_chunk0: Optional[torch.Tensor] = None   # [n_prefill + 1]
     chunk_row0: Optional[torch.Tensor] = None
     chunk_len: Optional[torch.Tensor] = None
+    # -- latent attention: rows 0..n_latent-1 attend in the latent space, the
+    # rest (the tile32 tiles) over keys and values made from these cache slots
+    n_latent: int = 0
+    ctx_slots: Optional[torch.Tensor] = None    # slots of their contexts
+    tile32_ctx0: Optional[torch.Tensor] = None  # where a tile's context starts
 
     @property
     def total_tokens(self) -> int:
@@ -83,8 +88,15 @@ class ForwardBatch:
             "tile_seq": self.tile32_seq, "tile_pos0": self.tile32_pos0,
             "state_slots": self.state_slots, "seg_row0": self.seg_row0,
             "seg_len": self.seg_len, "seg_chunk0": self.seg_chunk0,
-            "chunk_row0": self.chunk_row0, "chunk_len": self.chunk_len}
+            "chunk_row0": self.chunk_row0, "chunk_len": self.chunk_len,
+            "short_q0": self.tile_q0, "short_qn": self.tile_qn,
+            "short_seq": self.tile_seq, "short_pos0": self.tile_pos0,
+            "tile_ctx0": self.tile32_ctx0, "ctx_slots": self.ctx_slots}
         return {k: t for k, t in named.items() if t is not None}
+
+    def hybrid_numbers(self) -> Dict[str, int]:
+        return {"n_decode": self.n_decode, "n_latent": self.n_latent,
+                "max_ctx": self.max_ctx, "max_kv": self.max_kv}
 
 
 class KVCache:

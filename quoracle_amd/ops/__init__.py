@@ -54,9 +54,29 @@ def ext():
     return _require("_quoracle_ops")
 
 
+def module(name: str):
+    """A native module by its name; raises when missing."""
+    return _require(name)
+
+
 def hybrid_ext():
-    """The native module of the hybrid models; raises when missing."""
+    """The kernels of recurrent and chunk-local mixers; raises when missing."""
     return _require("_quoracle_hybrid")
+
+
+def latent_ext():
+    """The kernels of latent attention and of mixtures of experts; raises
+    when missing."""
+    return _require("_quoracle_latent")
+
+
+def stream_ext():
+    """A module with the embedding and final-norm kernels that all hybrid
+    models share: the one that is loaded, or any that is built."""
+    for name in ("_quoracle_latent", "_quoracle_hybrid"):
+        if name in _loaded:
+            return _loaded[name]
+    return _load("_quoracle_latent") or hybrid_ext()
 
 
 # -- thin wrappers -----------------------------------------------------------

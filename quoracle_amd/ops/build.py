@@ -1,10 +1,11 @@
 """In-tree hipcc build of the quoracle_amd HIP extensions (gfx950).
 
-Two modules, each one translation unit, built directly with hipcc (no JIT
+Three modules, each one translation unit, built directly with hipcc (no JIT
 cache — the .so files must travel with the repo snapshot to the GPU box):
 
   _quoracle_ops     the Llama-family kernels and their forward driver
   _quoracle_hybrid  recurrent/local-attention mixers and the hybrid driver
+  _quoracle_latent  latent attention, mixtures of experts and the same driver
 
 They are separate so that a process serving one family compiles and loads
 only that family's kernels.  hipcc cross-compiles gfx950 without a GPU, so
@@ -30,9 +31,15 @@ MODULES: Dict[str, Sequence[str]] = {
         "bindings.cpp", "common.h", "forward.h", "attention.hip",
         "attention_mfma.hip", "attention_core.h", "elementwise.hip"),
     "_quoracle_hybrid": (
-        "hybrid_bindings.cpp", "common.h", "hybrid_common.h", "attention_core.h",
-        "attention_local.hip", "linear_attention.hip",
-        "hybrid_elementwise.hip", "hybrid_forward.h"),
+        "hybrid_bindings.cpp", "common.h", "hybrid_common.h", "hybrid_host.h",
+        "stream_kernels.hip", "attention_core.h", "attention_local.hip",
+        "linear_attention.hip", "hybrid_elementwise.hip", "hybrid_forward.h",
+        "hybrid_blocks.h"),
+    "_quoracle_latent": (
+        "latent_bindings.cpp", "common.h", "hybrid_common.h", "hybrid_host.h",
+        "stream_kernels.hip", "latent_elementwise.hip", "grouped_gemm.hip",
+        "latent_attention.hip", "moe.hip", "hybrid_forward.h",
+        "latent_blocks.h"),
 }
 
 

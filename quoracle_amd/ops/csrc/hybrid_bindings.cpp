@@ -10,85 +10,14 @@
 #include <stdexcept>
 #include <string>
 
+#include "stream_kernels.hip"
 #include "attention_local.hip"
 #include "linear_attention.hip"
 #include "hybrid_elementwise.hip"
 
 namespace {
 
-using torch::Tensor;
-using OptTensor = c10::optional<Tensor>;
-
-hipStream_t current_stream() {
-  return c10::hip::getCurrentHIPStream().stream();
-}
-
-#define CHECK_GPU(t)                                                     \
-  TORCH_CHECK((t).is_cuda(), #t " must be on the GPU");                  \
-  TORCH_CHECK((t).is_contiguous(), #t " must be contiguous")
-#define CHECK_I32(t)                                                     \
-  CHECK_GPU(t);                                                          \
-  TORCH_CHECK((t).scalar_type() == torch::kInt32, #t " must be int32")
-#define CHECK_F32(t)                                                     \
-  CHECK_GPU(t);                                                          \
-  TORCH_CHECK((t).scalar_type() == torch::kFloat32, #t " must be float32")
-
-template <typename T> constexpr torch::ScalarType scalar_of();
-template <> constexpr torch::ScalarType scalar_of<bf16>() {
-  return torch::kBFloat16;
-}
-template <> constexpr torch::ScalarType scalar_of<float>() {
-  return torch::kFloat32;
-}
-template <typename T> T *ptr(const Tensor &t) {
-  TORCH_CHECK(t.scalar_type() == scalar_of<T>(), "mixed activation dtypes");
-  return reinterpret_cast<T *>(t.data_ptr());
-}
-const int *iptr(const Tensor &t) { return t.data_ptr<int>(); }
-float *fptr(const Tensor &t) { return t.data_ptr<float>(); }
-
-// Run `body` with T = the activation type of `t`.
-template <typename F> void by_dtype(const Tensor &t, F body) {
-  if (t.scalar_type() == torch::kBFloat16) body(bf16());
-  else if (t.scalar_type() == torch::kFloat32) body(float());
-  else TORCH_CHECK(false, "activations must be bfloat16 or float32");
-}
-template <int N> using Int = std::integral_constant<int, N>;
-template <typename F> void by_vec(bool vec8, F body) {
-  if (vec8) body(Int<8>());
-  else body(Int<1>());
-}
-// Register groups per thread of a 256-thread norm over n values; 0: too many.
-template <typename F> void by_items(int n, int vec, F body) {
-  const int need = (n + 256 * vec - 1) / (256 * vec);
-  if (need <= 1) body(Int<1>());
-  else if (need <= 2) body(Int<2>());
-  else if (need <= 4) body(Int<4>());
-  else body(Int<0>());
-}
-
-void embed_positions(Tensor x, Tensor h, Tensor embed, OptTensor table,
-                     Tensor tokens, Tensor positions) {
-  CHECK_F32(x); CHECK_GPU(h); CHECK_GPU(embed);
-  CHECK_I32(tokens); CHECK_I32(positions);
-  const int n = embed.size(1);
-  const long T = tokens.size(0);
-  TORCH_CHECK(x.numel() == T * n && h.numel() == T * n &&
-              positions.size(0) == T, "embed_positions shapes");
-  if (table) { CHECK_GPU(*table); TORCH_CHECK(table->size(1) == n, "table"); }
-  if (T == 0) return;
-  by_dtype(embed, [&](auto t0) {
-    using A = decltype(t0);
-    by_vec(n % 8 == 0, [&](auto v) {
-      embed_positions_kernel<A, decltype(v)::value>
-          <<<dim3(T), dim3(256), 0, current_stream()>>>(
-              fptr(x), ptr<A>(h), ptr<A>(embed),
-              table ? ptr<A>(*table) : nullptr, iptr(tokens), iptr(positions),
-              n);
-    });
-  });
-  HIP_CHECK_KERNEL();
-}
+#include "hybrid_host.h"
 
 void post_norm(Tensor x, Tensor h, Tensor a, double sa, OptTensor b,
                double sb, double alpha, Tensor w, double eps) {
@@ -109,26 +38,6 @@ void post_norm(Tensor x, Tensor h, Tensor a, double sa, OptTensor b,
                 b ? ptr<A>(*b) : nullptr, (float)sb, (float)alpha, fptr(w), n,
                 (float)eps);
       });
-    });
-  });
-  HIP_CHECK_KERNEL();
-}
-
-void norm_rows(Tensor out, Tensor x, Tensor rows, Tensor w, double eps) {
-  CHECK_GPU(out); CHECK_F32(x); CHECK_GPU(rows); CHECK_F32(w);
-  TORCH_CHECK(rows.scalar_type() == torch::kInt64, "rows must be int64");
-  const int n = w.size(0);
-  const long R = rows.size(0);
-  TORCH_CHECK(out.numel() == R * n && x.size(-1) == n, "norm_rows shapes");
-  if (R == 0) return;
-  by_dtype(out, [&](auto t0) {
-    using A = decltype(t0);
-    by_vec(n % 8 == 0, [&](auto v) {
-      norm_rows_kernel<A, decltype(v)::value>
-          <<<dim3(R), dim3(256), 0, current_stream()>>>(
-              ptr<A>(out), fptr(x),
-              reinterpret_cast<const long *>(rows.data_ptr<int64_t>()),
-              fptr(w), n, (float)eps);
     });
   });
   HIP_CHECK_KERNEL();
@@ -532,15 +441,13 @@ void linear_chunked(Tensor o, Tensor proj, int64_t q_off, int64_t k_off,
 }
 
 #include "hybrid_forward.h"
+#include "hybrid_blocks.h"
 
 }  // namespace
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.attr("LIN_CHUNK") = LIN_CHUNK;
-  m.def("embed_positions", &embed_positions,
-        "Token embedding plus learned positions into the float32 stream");
   m.def("post_norm", &post_norm, "Residual sum and RMS norm after it");
-  m.def("norm_rows", &norm_rows, "Final RMS norm of selected rows");
   m.def("glu", &glu, "SiLU(gate) * up");
   m.def("gated_norm", &gated_norm, "Grouped RMS norm times a gate");
   m.def("qk_norm_rope_store", &qk_norm_rope_store,
@@ -558,12 +465,5 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("linear_chunked", &linear_chunked,
         "Chunked linear attention on the matrix cores (bf16 prefill)");
   m.def("linear_tiles_ok", &linear_tiles_ok, "Chunked form applies");
-  m.def("register_hybrid", &qhybrid::register_model,
-        "Register a hybrid model's weights with the native driver");
-  m.def("unregister_hybrid", &qhybrid::unregister_model,
-        "Drop a registered model");
-  m.def("hybrid_forward", &qhybrid::forward,
-        "All layers of one mixed batch; returns the float32 stream");
-  m.def("hybrid_logits", &qhybrid::compute_logits,
-        "Final norm and head of selected rows");
+  qhybrid::bind(m);
 }

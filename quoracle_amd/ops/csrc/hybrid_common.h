@@ -88,4 +88,23 @@ __device__ __forceinline__ float activate(float z, int act) {
   return z;
 }
 
+// z * Phi(z), the exact (erf) gelu.  For values that are rounded to bf16
+// afterwards erf(|u|) = 1 - P(t) exp(-u^2), t = 1 / (1 + 0.3275911 |u|), with
+// P of degree five: Abramowitz and Stegun, Handbook of Mathematical Functions,
+// 7.1.26, absolute error below 1.5e-7.
+template <typename T> __device__ __forceinline__ float gelu(float z) {
+  const float u = z * 0.70710678f;
+  if constexpr (sizeof(T) == 2) {
+    const float t = __builtin_amdgcn_rcpf(fmaf(0.3275911f, fabsf(u), 1.f));
+    float p = fmaf(1.061405429f, t, -1.453152027f);
+    p = fmaf(p, t, 1.421413741f);
+    p = fmaf(p, t, -0.284496736f);
+    p = fmaf(p, t, 0.254829592f);
+    const float e = 1.f - p * t * __expf(-u * u);
+    return 0.5f * z * (1.f + copysignf(e, u));
+  } else {
+    return 0.5f * z * (1.f + erff(u));
+  }
+}
+
 }  // namespace hyb

@@ -14,7 +14,7 @@ from typing import Optional
 
 import torch
 
-from . import hybrid_ext
+from . import hybrid_ext, stream_ext
 from . import reference as ref
 
 LIN_CHUNK = 64          # tokens per linear-attention chunk (csrc LIN_CHUNK)
@@ -27,7 +27,7 @@ def embed_positions(x, h, embed, table: Optional[torch.Tensor], tokens,
                     positions) -> None:
     """x = embed[tokens] (+ table[positions]) in float32; h = x in h's type."""
     if x.is_cuda:
-        hybrid_ext().embed_positions(x, h, embed, table, tokens, positions)
+        stream_ext().embed_positions(x, h, embed, table, tokens, positions)
         return
     ref.embed_positions(x, h, embed, table, tokens, positions)
 
@@ -44,7 +44,7 @@ def post_norm(x, h, a, sa: float, b: Optional[torch.Tensor], sb: float,
 def norm_rows(out, x, rows, w, eps: float) -> None:
     """out[r] = rms(x[rows[r]]) * w."""
     if x.is_cuda:
-        hybrid_ext().norm_rows(out, x, rows, w, eps)
+        stream_ext().norm_rows(out, x, rows, w, eps)
         return
     ref.norm_rows(out, x, rows, w, eps)
 

@@ -256,3 +256,98 @@ def linear_attention(o, proj, q_off, k_off, v_off, act, qscale, decay,
         S.mul_(a[t][:, None, :]).add_(v[t][:, :, None] * k[t][:, None, :])
         y[t] = (S @ q[t][:, :, None]).squeeze(-1) * qscale
     o.copy_(y.view_as(o))
+
+
+# -- latent attention, mixtures of experts, norms around a sublayer ----------
+
+def pre_norm(x, h, y, w, eps) -> None:
+    if y is not None:
+        x.copy_(y)
+    h.copy_(_rms(x, w, eps))
+
+
+def sandwich_norm(x, h, joined, w_next, y, bias, y2, gate, w, eps) -> None:
+    s = y.float()
+    if s.dim() == 3:
+        s = s.sum(1)
+    if bias is not None:
+        s = s + bias
+    if y2 is not None:
+        s = s + gate[:, None] * y2.float()
+    x += _rms(s, w, eps)
+    if w_next is not None:
+        h.copy_(_rms(x, w_next, eps))
+    if joined is not None:
+        joined[:, :x.shape[1]] = x.to(joined.dtype)
+
+
+def latent_store(cq, pool, proj, kv_off, rank_p, wq, wkv, positions, slots,
+                 freq, eps) -> None:
+    bs = pool.shape[1]
+    rank, n = wkv.shape[0], 2 * freq.shape[0]
+    cq.copy_(_rms(proj[:, :wq.shape[0]].float(), wq, eps))
+    c = _rms(proj[:, kv_off:kv_off + rank].float(), wkv, eps)
+    k = rope_interleaved(
+        proj[:, None, kv_off + rank:kv_off + rank + n].float(), positions,
+        freq, 1.0)[:, 0]
+    row = torch.zeros(c.shape[0], pool.shape[2])
+    row[:, :rank] = c
+    row[:, rank_p:rank_p + n] = k
+    at = slots.long()
+    pool[at // bs, at % bs] = row.to(pool.dtype)
+
+
+def rotate_heads(q, off, positions, freq) -> None:
+    n = 2 * freq.shape[0]
+    part = q[..., off:off + n].float()
+    q[..., off:off + n] = rope_interleaved(part, positions, freq,
+                                           1.0).to(q.dtype)
+
+
+def latent_attention(out, q, pool, w_kv, sink, scale, block_tables, row_seq,
+                     positions) -> None:
+    T, H, V = out.shape
+    rot = pool.shape[2] - w_kv.shape[1]
+    dim = q.shape[2] - rot
+    rank = w_kv.shape[1]
+    w = w_kv.float()
+    for seq in row_seq.unique().tolist():
+        rows = (row_seq == seq).nonzero(as_tuple=True)[0]
+        pos = positions[rows].long()
+        length = int(pos.max()) + 1
+        blocks = block_tables[seq, :-(-length // pool.shape[1])].long()
+        ctx = pool[blocks].flatten(0, 1)[:length].float()
+        kv = ctx[:, :rank] @ w.T
+        k = torch.cat([kv[:, :H * dim].view(length, H, dim),
+                       ctx[:, None, rank:].expand(length, H, rot)], -1)
+        v = kv[:, H * dim:].view(length, H, V)
+        s = torch.einsum("qhd,khd->hqk", q[rows].float(), k) * scale
+        s = s.masked_fill(torch.arange(length)[None, None, :]
+                          > pos[None, :, None], float("-inf"))
+        if sink is not None:
+            s = torch.cat([s, sink[:, None, None].expand(H, len(rows), 1)],
+                          dim=-1)
+        p = torch.softmax(s, dim=-1)[..., :length]
+        out[rows] = torch.einsum("hqk,khd->qhd", p, v).to(out.dtype)
+
+
+def bias_gelu(up, bias) -> None:
+    v = up.float() if bias is None else up.float() + bias
+    up.copy_(torch.nn.functional.gelu(v))
+
+
+def moe_route(ids, weights, gate, h, router, experts) -> None:
+    s = torch.sigmoid(h.float() @ router.float().T)
+    w, i = s[:, :experts].topk(ids.shape[1], dim=-1)
+    ids.copy_(i)
+    weights.copy_(w)
+    if gate is not None:
+        gate.copy_(s[:, experts])
+
+
+def moe_experts(y, h, ids, weights, up, down) -> None:
+    for e in ids.unique().tolist():
+        t, k = (ids == e).nonzero(as_tuple=True)
+        z = (h[t].float() @ up[e].float().T) * weights[t, k, None]
+        a = torch.nn.functional.gelu(z)
+        y[t, k] = (a @ down[e].float().T).to(y.dtype)

@@ -345,8 +345,12 @@ void latent_attend(const Tensor &out, const Tensor &q, const Tensor &pool,
   TORCH_CHECK(d.rank % 8 == 0 && d.rot % 8 == 0 && d.dim % 8 == 0 &&
               d.vdim % 8 == 0, "latent attention sizes are padded to 8");
   if (sink) { CHECK_F32(*sink); TORCH_CHECK(sink->numel() == d.H, "sink"); }
+  // a batch with portions that names neither short tiles nor contexts is one
+  // of a model with other layers that the matrix kernels do not take
   const bool tiles = q.scalar_type() == torch::kBFloat16 && d.rank <= 512 &&
-                     d.rot <= 64;
+                     d.rot <= 64 &&
+                     (T == b.n_decode || b.n_latent > b.n_decode ||
+                      b.has("ctx_slots"));
   const long n = tiles ? b.n_latent : T;
   TORCH_CHECK(b.n_decode <= n && n <= T, "latent attention rows");
   auto w_uv = w_kv.narrow(0, (long)d.H * d.dim, (long)d.H * d.vdim)

@@ -1,13 +1,10 @@
-"""Small Koridra configurations with random weights, and helpers that feed
-them to the engine and to the plain oracle."""
+"""Small Koridra configurations with random weights."""
 
-import json
 import math
-import os
-import struct
 
 import torch
 
+import hybrid_cases
 import koridra_oracle as oracle
 
 # name -> configuration; sizes are chosen so that nothing is equal by chance
@@ -129,94 +126,8 @@ def random_weights(cfg, rank, seed=0):
     return {k: v.to(torch.bfloat16) for k, v in t.items()}
 
 
-def write_checkpoint(folder, cfg, weights):
-    """config.json + model.safetensors."""
-    os.makedirs(folder, exist_ok=True)
-    with open(os.path.join(folder, "config.json"), "w") as f:
-        json.dump(cfg, f)
-    header, blobs, at = {}, [], 0
-    for name, w in weights.items():
-        raw = w.contiguous().view(torch.int16).numpy().tobytes()
-        header[name] = {"dtype": "BF16", "shape": list(w.shape),
-                        "data_offsets": [at, at + len(raw)]}
-        blobs.append(raw)
-        at += len(raw)
-    head = json.dumps(header).encode()
-    with open(os.path.join(folder, "model.safetensors"), "wb") as f:
-        f.write(struct.pack("<Q", len(head)) + head + b"".join(blobs))
-    return folder
-
-
-def tokens_for(cfg, n, seed):
-    return torch.randint(0, cfg["vocab"], (n,),
-                         generator=torch.Generator().manual_seed(seed)).tolist()
-
-
-class Case:
-    """One configuration on disk, its weights, and remembered oracle logits."""
-
+class Case(hybrid_cases.Case):
     def __init__(self, name, folder, cfg=None, seed=0):
-        self.name = name
-        self.cfg = cfg or CONFIGS[name]
-        self.weights = random_weights(self.cfg, RANKS.get(name, 4), seed)
-        self.path = write_checkpoint(str(folder), self.cfg, self.weights)
-        self._known = {}
-
-    def logits(self, tokens):
-        key = tuple(tokens)
-        if key not in self._known:
-            self._known[key] = oracle.forward(self.cfg, self.weights,
-                                              tokens)[0]
-        return self._known[key]
-
-    def engine(self, device, dtype, blocks=96, slots=4, **kw):
-        from quoracle_amd.engine.engine import LocalEngine
-        return LocalEngine([self.path], device=torch.device(device),
-                           embed_model_key=None, kv_blocks_override=blocks,
-                           dtype=dtype, state_slots=slots, **kw)
-
-
-def error(got, want):
-    """Largest per-row RMS difference, in units of the logits' RMS."""
-    got, want = got.double(), want.double()
-    d = (got - want).square().mean(-1).sqrt()
-    return float(d.max() / want.square().mean().sqrt())
-
-
-def tolerance(dtype):
-    return 2e-5 if dtype == torch.float32 else 0.06
-
-
-def feed(engine, path, schedule):
-    """Run [[(id, tokens), ...], ...] with every place wanted; returns
-    {id: logits of all its tokens so far}.  A request ends when its id is
-    given as (id, None)."""
-    out, live = {}, set()
-    for step in schedule:
-        ends = [i for i, toks in step if toks is None]
-        parts = [(i, toks) for i, toks in step if toks]
-        live.update(i for i, _ in parts)
-        if parts:
-            lg = engine.step_entries(
-                path, [(i, toks, range(len(toks))) for i, toks in parts],
-                live)
-            at = 0
-            for i, toks in parts:
-                out.setdefault(i, []).append(lg[at:at + len(toks)])
-                at += len(toks)
-        for i in ends:
-            engine.drop_session(path, i)
-            live.discard(i)
-    return {i: torch.cat(p) for i, p in out.items()}
-
-
-def cut(tokens, sizes):
-    """Split tokens into portions of the given sizes, cycling."""
-    parts, at, k = [], 0, 0
-    while at < len(tokens):
-        n = sizes[k % len(sizes)]
-        parts.append(tokens[at:at + n])
-        at, k = at + n, k + 1
-    return parts
-
-
+        cfg = cfg or CONFIGS[name]
+        super().__init__(name, folder, cfg,
+                         random_weights(cfg, RANKS.get(name, 4), seed), oracle)

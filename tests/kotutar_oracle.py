@@ -24,15 +24,15 @@ def gelu(z):
 
 
 def rotate(x, position, dims, base):
-    """Turn the pairs (2i, 2i+1), i < dims / 2, of one vector by
+    """Turn the pairs (2i, 2i+1), i < dims / 2, of the last axis by
     position * base^(-2i/dims); what lies behind them passes."""
     y = x.clone()
     for i in range(dims // 2):
         a = position * base ** (-2.0 * i / dims)
         c, s = math.cos(a), math.sin(a)
-        u, v = x[2 * i], x[2 * i + 1]
-        y[2 * i] = u * c - v * s
-        y[2 * i + 1] = v * c + u * s
+        u, v = x[..., 2 * i], x[..., 2 * i + 1]
+        y[..., 2 * i] = u * c - v * s
+        y[..., 2 * i + 1] = v * c + u * s
     return y
 
 
@@ -41,23 +41,22 @@ def sees(i, j):
 
 
 def sink_softmax(scores, sink):
-    """Weights of the scores when exp(sink) joins the denominator."""
-    top = max(float(scores.max()), float(sink))
+    """Weights of the scores [n, H] over n when exp(sink) [H] joins the
+    denominator."""
+    top = torch.maximum(scores.max(0).values, sink)
     e = torch.exp(scores - top)
-    return e / (math.exp(float(sink) - top) + e.sum())
+    return e / (torch.exp(sink - top) + e.sum(0))
 
 
 def attend(q, keys, values, scale, sink, positions=None):
     """q [Tq, H, D] at `positions` (default 0..) over keys [T, H, D] and
     values [T, H, V]; sink [H]."""
     positions = range(q.shape[0]) if positions is None else positions
-    H = q.shape[1]
-    out = torch.zeros(q.shape[0], H, values.shape[2], dtype=q.dtype)
+    out = torch.zeros(q.shape[0], q.shape[1], values.shape[2], dtype=q.dtype)
     for r, i in enumerate(positions):
         js = [j for j in range(keys.shape[0]) if sees(i, j)]
-        for h in range(H):
-            s = (keys[js, h] @ q[r, h]) * scale
-            out[r, h] = sink_softmax(s, sink[h]) @ values[js, h]
+        w = sink_softmax((keys[js] * q[r]).sum(-1) * scale, sink)
+        out[r] = (w[:, :, None] * values[js]).sum(0)
     return out
 
 
@@ -79,8 +78,7 @@ def latent_queries(h, W, p, m, eps, positions=None):
     q = rms_norm(h @ W[p + "dq"].T, W[p + "dq.norm"], eps) @ W[p + "uq"].T
     q = q.view(T, H, D + n).clone()
     for t, i in enumerate(positions):
-        for a in range(H):
-            q[t, a, D:] = rotate(q[t, a, D:], i, n, m["rot"]["base"])
+        q[t, :, D:] = rotate(q[t, :, D:], i, n, m["rot"]["base"])
     return q
 
 

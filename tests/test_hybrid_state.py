@@ -6,7 +6,8 @@ import struct
 import pytest
 import torch
 
-from koridra_cases import CONFIGS, RANKS, random_weights, write_checkpoint
+from hybrid_cases import write_checkpoint
+from koridra_cases import CONFIGS, RANKS, random_weights
 from quoracle_amd.engine.kv_cache import (BlockManager, OutOfBlocks,
                                           OutOfSlots, SessionCache, StateSlots)
 from quoracle_amd.models import KoridraModel, build_model, get_config

@@ -12,8 +12,9 @@ import pytest
 import torch
 
 import koridra_oracle as oracle
-from koridra_cases import (CONFIGS, Case, cut, error, feed, tokens_for,
-                           tolerance)
+from hybrid_cases import (cut, error, feed, greedy, paced, request, tokens_for,
+                          tolerance)
+from koridra_cases import CONFIGS, Case
 
 REPO = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 WHERE = [
@@ -96,21 +97,7 @@ def test_mixed_batches_and_reuse(cases, name, where):
              "e": cut(reqs["e"], [16]), "f": cut(reqs["f"], [1, 31])}
     eng = case.engine(*where, blocks=20, slots=3)
     eng.precapture_graphs((1, 2, 4))
-    steps, waiting, live, turn = [], list(lens), [], 0
-    while waiting or live:
-        while waiting and len(live) < 3:
-            live.append(waiting.pop(0))
-        step = []
-        for i, r in enumerate(list(live)):
-            if (turn + i) % 4 == 3 and len(live) > 1:
-                continue                     # left out of this step
-            step.append((r, parts[r].pop(0)))
-            if not parts[r]:
-                step.append((r, None))
-                live.remove(r)
-        steps.append(step)
-        turn += 1
-    got = feed(eng, case.path, steps)
+    got = feed(eng, case.path, paced(parts, 3))
     check(case, got, reqs, where[1])
     hm = eng.models[case.path]
     assert hm.mgr.free_blocks == 19 and hm.sessions.states.free_slots == 3
@@ -200,22 +187,6 @@ def test_oracle_shows_a_wrong_mechanism(cases, mechanism):
 
 # -- generation --------------------------------------------------------------
 
-def _greedy(case, prompt, n):
-    out = []
-    for _ in range(n):
-        lg, _ = oracle.forward(case.cfg, case.weights, prompt + out)
-        out.append(int(lg[-1].argmax()))
-        if out[-1] == 257:                       # end of sequence
-            break
-    return out
-
-
-def _request(case, text, n, **kw):
-    from quoracle_amd.engine.api import GenerateRequest
-    return GenerateRequest(model_key=case.path, temperature=0.0, max_tokens=n,
-                           messages=[{"role": "user", "content": text}], **kw)
-
-
 @pytest.mark.parametrize("where", WHERE[:2])
 @pytest.mark.parametrize("chunk", [2048, 7])
 def test_greedy_generation(cases, where, chunk):
@@ -225,8 +196,8 @@ def test_greedy_generation(cases, where, chunk):
     eng = case.engine(*where, prefill_chunk=chunk)
     prompt = eng.tokenizer.render_messages(
         [{"role": "user", "content": "a chunk border lies in this"}])
-    want = _greedy(case, prompt, 12)
-    r = eng.generate_sync(_request(case, "a chunk border lies in this", 12),
+    want = greedy(case, prompt, 12)
+    r = eng.generate_sync(request(case, "a chunk border lies in this", 12),
                           timeout=120)
     assert r.ok, r.error
     assert r.output_tokens == len(want)
@@ -242,11 +213,11 @@ def test_more_requests_than_slots(cases, where):
     alone = {}
     for t in texts:
         alone[t] = case.engine(*where).generate_sync(
-            _request(case, t, 9), timeout=120).text
+            request(case, t, 9), timeout=120).text
     eng = case.engine(*where, slots=2)
     done = {}
     for t in texts:
-        eng._submit(_request(case, t, 9),
+        eng._submit(request(case, t, 9),
                     ("cb", lambda r, t=t: done.__setitem__(t, r)))
     for _ in range(400):
         if len(done) == len(texts):
@@ -264,12 +235,12 @@ def test_session_continues_or_starts_over(cases, where):
     fresh engine."""
     case = cases("odd")
     eng = case.engine(*where)
-    first = eng.generate_sync(_request(case, "hello", 6, session_id="s"),
+    first = eng.generate_sync(request(case, "hello", 6, session_id="s"),
                               timeout=120)
     sess = eng.models[case.path].sessions.get_or_create("s")
     held = list(sess.token_ids)
     # same prompt again: its state has moved past the prompt, so start over
-    again = eng.generate_sync(_request(case, "hello", 6, session_id="s"),
+    again = eng.generate_sync(request(case, "hello", 6, session_id="s"),
                               timeout=120)
     assert again.text == first.text
     assert eng.stats["prefix_hit_tokens"] == 0
@@ -277,9 +248,9 @@ def test_session_continues_or_starts_over(cases, where):
     sid = eng.models[case.path].sessions
     assert sid.match_prefix(sess, held + [1, 2]) == len(held)
     # another text in the same session
-    other = eng.generate_sync(_request(case, "help", 6, session_id="s"),
+    other = eng.generate_sync(request(case, "help", 6, session_id="s"),
                               timeout=120)
-    fresh = case.engine(*where).generate_sync(_request(case, "help", 6),
+    fresh = case.engine(*where).generate_sync(request(case, "help", 6),
                                               timeout=120)
     assert other.text == fresh.text
 
@@ -289,7 +260,7 @@ def test_idle_sessions_make_room(cases):
     case = cases("odd")
     eng = case.engine("cpu", torch.float32, slots=1)
     for name in ("x", "y", "x"):
-        r = eng.generate_sync(_request(case, name, 3, session_id=name),
+        r = eng.generate_sync(request(case, name, 3, session_id=name),
                               timeout=60)
         assert r.ok, r.error
 
@@ -314,17 +285,17 @@ def test_failed_step_drops_its_sessions(cases, monkeypatch):
     trusted: the next request of the session starts over."""
     case = cases("odd")
     eng = case.engine("cpu", torch.float32)
-    want = eng.generate_sync(_request(case, "abc", 4), timeout=60).text
+    want = eng.generate_sync(request(case, "abc", 4), timeout=60).text
     hm = eng.models[case.path]
     good = hm.model.forward
     monkeypatch.setattr(hm.model, "forward",
                         lambda *a, **k: (_ for _ in ()).throw(
                             RuntimeError("planted")))
-    r = eng.generate_sync(_request(case, "abc", 4, session_id="s"),
+    r = eng.generate_sync(request(case, "abc", 4, session_id="s"),
                           timeout=60)
     assert not r.ok
     monkeypatch.setattr(hm.model, "forward", good)
-    r = eng.generate_sync(_request(case, "abc", 4, session_id="s"),
+    r = eng.generate_sync(request(case, "abc", 4, session_id="s"),
                           timeout=60)
     assert r.ok and r.text == want
 
@@ -426,5 +397,5 @@ def test_generate_command(cases):
         cwd=REPO, capture_output=True, text=True, timeout=240)
     assert p.returncode == 0, p.stderr[-2000:]
     want = case.engine("cpu", torch.float32).generate_sync(
-        _request(case, "hi", 5), timeout=60)
+        request(case, "hi", 5), timeout=60)
     assert p.stdout.rstrip("\n") == want.text.rstrip("\n")

@@ -57,10 +57,16 @@ def parse_args():
                         "llama3-70b+mixtral-8x7b)")
     p.add_argument("--layer-bench", action="store_true",
                    help="instead of the flagship workload: prefill and "
-                        "decode throughput of Koridra layers beside Llama "
-                        "layers of equal size, one JSON line each")
-    p.add_argument("--layer-bench-only", choices=["koridra", "llama"],
-                   default=None, help="one side of --layer-bench (profiling)")
+                        "decode throughput of the hybrid models' layers beside "
+                        "Llama and Mixtral layers of equal size, one JSON "
+                        "line each")
+    p.add_argument("--layer-bench-only", nargs="+", default=None,
+                   choices=["llama", "koridra", "kotutar", "mixtral",
+                            "kotutar-moe"],
+                   help="some models of --layer-bench (profiling)")
+    p.add_argument("--layer-bench-size", nargs="+", default=None,
+                   choices=["1b-layers", "8b-layers"],
+                   help="some sizes of --layer-bench")
     return p.parse_args()
 
 
@@ -82,7 +88,9 @@ def main():
           file=sys.stderr, flush=True)
     if args.layer_bench:
         from quoracle_amd.tools import layer_bench
-        layer_bench.main(device=args.device, only=args.layer_bench_only)
+        layer_bench.main(device=args.device, only=args.layer_bench_only,
+                         **({"sizes": args.layer_bench_size}
+                            if args.layer_bench_size else {}))
         return
 
     rank = int(os.environ.get("RANK", "0"))

@@ -1,11 +1,14 @@
-"""Prefill and decode throughput of a hybrid model beside a Llama-family model
-of equal size, through the engine's own step.
+"""Prefill and decode throughput of the hybrid models beside Llama-family
+models of equal size, through the engine's own step.
 
   python bench.py --layer-bench            (one JSON line per measurement)
 
 Random weights; a few layers of the size of a 1B-class and of an 8B-class
 model, so that a step is long enough to time and short enough to repeat.  The
-two models take turns.
+models take turns.  Beside Llama stand Koridra and Kotutar with dense
+feed-forwards, beside Mixtral (Llama with experts) Kotutar with experts.
+Kotutar's feed-forwards have two matrices for Llama's three and are as much
+wider.
 """
 
 from __future__ import annotations
@@ -23,6 +26,7 @@ SIZES = {
     "1b-layers": (2048, 8192, 8, 16, 4, 128),
     "8b-layers": (4096, 14336, 8, 32, 8, 128),
 }
+EXPERTS, TOP = 8, 2
 VOCAB = 32000
 CONTEXT = 16384
 ATTN_CHUNK = 8192
@@ -30,17 +34,29 @@ ATTN_CHUNK = 8192
 
 def configs(size: str) -> Dict[str, object]:
     from ..models.config import PRESETS
-    from ..models.hybrid_config import koridra_preset
+    from ..models.hybrid_config import koridra_preset, kotutar_preset
     hidden, ff, layers, heads, kv, dim = SIZES[size]
+    llama = replace(PRESETS["llama3-8b"], name=f"llama-{size}",
+                    vocab_size=VOCAB, n_layers=layers, hidden=hidden,
+                    n_heads=heads, n_kv_heads=kv, head_dim=dim,
+                    intermediate=ff, max_context=CONTEXT)
+
+    def kotutar(name: str, every: int):
+        return kotutar_preset(
+            f"{name}-{size}", vocab=VOCAB, hidden=hidden, n_layers=layers,
+            ff=ff * 3 // 2, heads=heads, dim=dim, rot_dim=dim // 2, vdim=dim,
+            q_rank=hidden * 3 // 8, kv_rank=512, experts=EXPERTS, top=TOP,
+            expert_ff=ff * 3 // 2, every=every, max_context=CONTEXT)
     return {
-        "llama": replace(PRESETS["llama3-8b"], name=f"llama-{size}",
-                         vocab_size=VOCAB, n_layers=layers, hidden=hidden,
-                         n_heads=heads, n_kv_heads=kv, head_dim=dim,
-                         intermediate=ff, max_context=CONTEXT),
+        "llama": llama,
         "koridra": koridra_preset(
             f"koridra-{size}", vocab=VOCAB, hidden=hidden, n_layers=layers,
             ff=ff, heads=heads, kv_heads=kv, dim=dim, chunk=ATTN_CHUNK,
             lin_heads=heads, lin_dim=dim, lin_vdim=dim, max_context=CONTEXT),
+        "kotutar": kotutar("kotutar", 0),
+        "mixtral": replace(llama, name=f"mixtral-{size}", n_experts=EXPERTS,
+                           top_k_experts=TOP),
+        "kotutar-moe": kotutar("kotutar-moe", 1),
     }
 
 
@@ -122,9 +138,9 @@ def main(sizes=tuple(SIZES), batches=(1, 16, 64), device=None,
          only=None) -> None:
     device = torch.device(device or "cuda:0")
     for size in sizes:
-        # interleave: both models live on the GPU at once
+        # interleave: all models live on the GPU at once
         sides = [Side(n, c, device, max(batches))
-                 for n, c in configs(size).items() if only in (None, n)]
+                 for n, c in configs(size).items() if not only or n in only]
         for s in sides:
             s.engine.precapture_graphs(tuple(batches))
 

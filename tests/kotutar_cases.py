@@ -52,7 +52,7 @@ CONFIGS = {
     # so short prompts are never expanded
     "small": config(
         290, 40, 1e-4, {"start": 0, "stop": 1, "times": 1},
-        (mixer(1, 16, 2, 16, 8, 8, 0.5, 77.0), moe(1, 1, 24)),
+        (mixer(1, 16, 2, 16, 8, 8, 0.22, 77.0), moe(1, 1, 24)),
         (mixer(2, 32, 16, 64, 24, 16, 0.2, 1e4), dense(56))),
     # many heads and experts, the largest head sizes of the prefill tiles, the
     # last layer is part of the loop

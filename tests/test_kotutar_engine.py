@@ -146,9 +146,10 @@ def test_short_and_long_portions_in_one_batch(cases, where):
     case = cases("tiles")
     eng = case.engine(*where)
     split = eng.models[case.path].model.expand_from or 20
-    assert 2 < split < 60
+    assert 2 < split < 100
     lens = {"a": split, "b": 1, "c": split - 1, "d": 2 * split, "e": 2}
-    reqs = {r: tokens_for(case.cfg, n + 40, n) for r, n in lens.items()}
+    reqs = {r: tokens_for(case.cfg, n + split + 9, n)
+            for r, n in lens.items()}
     got = feed(eng, case.path, [
         [(r, reqs[r][:n]) for r, n in lens.items()],
         [(r, reqs[r][n:n + k]) for (r, n), k

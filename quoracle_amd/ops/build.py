@@ -75,6 +75,7 @@ def _command(module: str, out: str) -> List[str]:
         # know the feature; that is harmless)
         "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
         "-Wno-unused-result",
+        "-Wno-inline-asm",      # M0 among the clobbers is meant
     ]
     for inc in includes + [py_include, CSRC]:
         cmd.append(f"-I{inc}")

@@ -4,15 +4,15 @@
 //
 //   B [groups][N][K] row-major, so both operands are contiguous along K.
 //   bf16 with K, the strides and the group offsets multiples of 8: MFMA
-//     gg_tile_kernel    BM x 128 tiles staged through LDS (many rows)
+//     gg_tile_kernel    tiles copied straight into LDS (many rows)
 //     gg_strip_kernel   16 rows x 32 columns per wave, operands straight from
 //                       memory; the waves share the columns' K range (weights
 //                       are read once, decode) or take columns side by side
 //   anything else, and float32: gg_plain_kernel.
 //
 // Rows.  Without a tile list blockIdx.z is the group and it has M rows.  With
-// one, blockIdx.y is a tile: group, first row and number of rows, 0 for tiles
-// that are not there.  `rows` maps a row of the sorted order to a slot
+// one, a workgroup takes a tile of it: group, first row and number of rows, 0
+// for tiles that are not there; tile_count says how many are.  `rows` maps a row of the sorted order to a slot
 // (token * top + k): A's row is then slot / a_div (a_div > 0) or the row
 // itself, C's row the slot (c_slot) or the row itself, and scale[slot]
 // multiplies the product before the gelu.
@@ -30,7 +30,8 @@ struct GroupedGemm {
   long lda, ldc;
   long a_group, c_group;               // element offset of a group's columns
   int M, N, K;
-  const int *tile_group, *tile_row0, *tile_rows;
+  const int *tile_group, *tile_row0, *tile_rows, *tile_count;
+  int row_tiles;                       // tiles of the list, or of a group
   const int *rows;
   int a_div;
   bool c_slot;
@@ -44,12 +45,10 @@ struct Tile {
   int group, row0, rows;
 };
 
-__device__ __forceinline__ Tile tile_of(const GroupedGemm &p, int BM) {
-  if (p.tile_group) {
-    const int i = blockIdx.y;
+__device__ __forceinline__ Tile tile_of(const GroupedGemm &p, int BM, int i) {
+  if (p.tile_group)
     return {p.tile_group[i], p.tile_row0[i], p.tile_rows[i]};
-  }
-  const int row0 = blockIdx.y * BM;
+  const int row0 = i * BM;
   return {(int)blockIdx.z, row0, min(BM, p.M - row0)};
 }
 
@@ -79,111 +78,116 @@ __device__ __forceinline__ float finish(const GroupedGemm &p, float v,
 
 }  // namespace gg
 
+// 16 bytes of zeros, copied where a row ends before a step does.
+__device__ const uint4 gg_zeros = {0, 0, 0, 0};
+
 // ---------------------------------------------------------------------------
-// BM x 128 tile, 64 deep, double-buffered in LDS; four waves of (BM/2) x 64.
-// Grid: (ceil(N/128), tiles, groups); block 256.
+// BM x BN tile, 64 deep, two buffers in LDS; WM x WN waves.  Rows of 64 values
+// in LDS hold their vector v at v ^ swizzle(row), so that the rows of a column
+// do not meet in a bank.  Each die takes a run of neighbouring tiles, four row
+// tiles before the next columns: they share an expert's rows and weights.
+// Grid: (ceil(N/BN) * tiles, 1, groups); block 64 * WM * WN.
 // ---------------------------------------------------------------------------
-template <int BM>
-__global__ void __launch_bounds__(256, 2) gg_tile_kernel(GroupedGemm p) {
-  constexpr int BN = 128, BK = 64, LS = BK + 8;
-  constexpr int NA = BM * BK / 8 / 256, NBV = BN * BK / 8 / 256;
-  constexpr int MI = BM / 64;                  // 32-row blocks of a wave
-  __shared__ __align__(16) bf16 a_s[2][BM * LS];
-  __shared__ __align__(16) bf16 b_s[2][BN * LS];
-  const gg::Tile tile = gg::tile_of(p, BM);
+template <int BM, int BN, int WM, int WN>
+__global__ void __launch_bounds__(64 * WM * WN, 2)
+gg_tile_kernel(GroupedGemm p) {
+  constexpr int BK = 64, NW = WM * WN, G = 4;
+  constexpr int MI = BM / WM / 32, NJ = BN / WN / 32;
+  constexpr int IA = BM / 8 / NW, IB = BN / 8 / NW;   // copies of 8 rows
+  __shared__ __align__(16) bf16 a_s[2][BM * BK];
+  __shared__ __align__(16) bf16 b_s[2][BN * BK];
+  const int cols = (p.N + BN - 1) / BN;
+  const int n_rows = p.tile_count ? *p.tile_count : p.row_tiles;
+  const int total = n_rows * cols;
+  int at = blockIdx.x;
+  if (at >= total) return;
+  {
+    const int die = at % 8, rest = total % 8;
+    at = die * (total / 8) + min(die, rest) + at / 8;
+  }
+  const int band = at / (G * cols), in = at % (G * cols);
+  const int high = min(G, n_rows - band * G);
+  const gg::Tile tile = gg::tile_of(p, BM, band * G + in % high);
   if (tile.rows <= 0) return;
-  const int n0 = blockIdx.x * BN;
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-  const int wm = wave >> 1, wn = wave & 1;
+  const int n0 = in / high * BN;
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int wm = wave / WN, wn = wave % WN;
   const int l31 = lane & 31, half = lane >> 5;
   const bf16 *a = (const bf16 *)p.a + tile.group * p.a_group;
   const bf16 *b = (const bf16 *)p.b + (long)tile.group * p.N * p.K;
 
-  const bf16 *a_at[NA], *b_at[NBV];            // null: rows that are not there
+  // copy i of this wave: rows 8 * (wave + i * NW) + lane / 8 (the last one
+  // again behind it), at kv of a step
+  static_assert(NW % 2 == 0, "rows of a copy keep their swizzle");
+  const int lr = lane >> 3;
+  const int kv = ((lane & 7) ^ ((wave * 8 + lr) >> 1 & 7)) * 8;
+  const bf16 *ap[IA], *bp[IB];
 #pragma unroll
-  for (int i = 0; i < NA; ++i) {
-    const int r = (tid + i * 256) / (BK / 8);
-    a_at[i] = r < tile.rows
-                  ? a + gg::a_row(p, tile.row0 + r) * p.lda + tid % 8 * 8
-                  : nullptr;
+  for (int i = 0; i < IA; ++i) {
+    const int r = min((wave + i * NW) * 8 + lr, tile.rows - 1);
+    ap[i] = a + gg::a_row(p, tile.row0 + r) * p.lda + kv;
   }
 #pragma unroll
-  for (int i = 0; i < NBV; ++i) {
-    const int r = (tid + i * 256) / (BK / 8);
-    b_at[i] = n0 + r < p.N ? b + (long)(n0 + r) * p.K + tid % 8 * 8 : nullptr;
+  for (int i = 0; i < IB; ++i) {
+    const int r = min(n0 + (wave + i * NW) * 8 + lr, p.N - 1);
+    bp[i] = b + (long)r * p.K + kv;
   }
-  uint4 ar[NA], br[NBV];
-  auto load = [&](int k0) {
-    const bool in = k0 + tid % 8 * 8 < p.K;
+  auto fetch = [&](int k0, int buf) {
+    const bool there = k0 + kv < p.K;
 #pragma unroll
-    for (int i = 0; i < NA; ++i)
-      ar[i] = in && a_at[i] ? *reinterpret_cast<const uint4 *>(a_at[i] + k0)
-                            : make_uint4(0, 0, 0, 0);
+    for (int i = 0; i < IA; ++i)
+      hyb::dma16(there ? (const void *)(ap[i] + k0) : &gg_zeros,
+                 &a_s[buf][(wave + i * NW) * 512]);
 #pragma unroll
-    for (int i = 0; i < NBV; ++i)
-      br[i] = in && b_at[i] ? *reinterpret_cast<const uint4 *>(b_at[i] + k0)
-                            : make_uint4(0, 0, 0, 0);
+    for (int i = 0; i < IB; ++i)
+      hyb::dma16(there ? (const void *)(bp[i] + k0) : &gg_zeros,
+                 &b_s[buf][(wave + i * NW) * 512]);
   };
-  auto stage = [&](int buf) {
-#pragma unroll
-    for (int i = 0; i < NA; ++i) {
-      const int j = tid + i * 256;
-      *reinterpret_cast<uint4 *>(&a_s[buf][j / 8 * LS + j % 8 * 8]) = ar[i];
-    }
-#pragma unroll
-    for (int i = 0; i < NBV; ++i) {
-      const int j = tid + i * 256;
-      *reinterpret_cast<uint4 *>(&b_s[buf][j / 8 * LS + j % 8 * 8]) = br[i];
-    }
-  };
-  gg_f32x16 acc[MI][2];
+  gg_f32x16 acc[MI][NJ];
 #pragma unroll
   for (int i = 0; i < MI; ++i)
 #pragma unroll
-    for (int j = 0; j < 2; ++j)
+    for (int j = 0; j < NJ; ++j)
 #pragma unroll
       for (int r = 0; r < 16; ++r) acc[i][j][r] = 0.f;
 
-  load(0);
-  stage(0);
-  __syncthreads();
+  fetch(0, 0);
+  const int sw = l31 >> 1 & 7;
   for (int k0 = 0, buf = 0; k0 < p.K; k0 += BK, buf ^= 1) {
-    const bool more = k0 + BK < p.K;
-    if (more) load(k0 + BK);
+    // also: the other buffer's readers are done
+    hyb::dma_barrier();
+    if (k0 + BK < p.K) fetch(k0 + BK, buf ^ 1);
+    const bf16 *as = &a_s[buf][(wm * (BM / WM) + l31) * BK];
+    const bf16 *bs = &b_s[buf][(wn * (BN / WN) + l31) * BK];
 #pragma unroll
     for (int kk = 0; kk < BK / 16; ++kk) {
-      gg_b16x8 af[MI], bfr[2];
+      const int v = ((kk * 2 + half) ^ sw) * 8;
+      gg_b16x8 af[MI], bfr[NJ];
 #pragma unroll
       for (int i = 0; i < MI; ++i)
-        af[i] = *reinterpret_cast<const gg_b16x8 *>(
-            &a_s[buf][(wm * (BM / 2) + i * 32 + l31) * LS + kk * 16 +
-                      half * 8]);
+        af[i] = *reinterpret_cast<const gg_b16x8 *>(as + i * 32 * BK + v);
 #pragma unroll
-      for (int j = 0; j < 2; ++j)
-        bfr[j] = *reinterpret_cast<const gg_b16x8 *>(
-            &b_s[buf][(wn * 64 + j * 32 + l31) * LS + kk * 16 + half * 8]);
+      for (int j = 0; j < NJ; ++j)
+        bfr[j] = *reinterpret_cast<const gg_b16x8 *>(bs + j * 32 * BK + v);
 #pragma unroll
       for (int i = 0; i < MI; ++i)
 #pragma unroll
-        for (int j = 0; j < 2; ++j)
+        for (int j = 0; j < NJ; ++j)
           acc[i][j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(
               af[i], bfr[j], acc[i][j], 0, 0, 0);
     }
-    // the other buffer: its readers passed the barrier of the last step
-    if (more) stage(buf ^ 1);
-    __syncthreads();
   }
 #pragma unroll
   for (int i = 0; i < MI; ++i)
 #pragma unroll
     for (int r = 0; r < 16; ++r) {
-      const int row = wm * (BM / 2) + i * 32 + (r & 3) + 8 * (r >> 2) +
+      const int row = wm * (BM / WM) + i * 32 + (r & 3) + 8 * (r >> 2) +
                       4 * half;
       if (row >= tile.rows) continue;
       const gg::Out o = gg::out_row(p, tile, tile.row0 + row);
 #pragma unroll
-      for (int j = 0; j < 2; ++j) {
-        const int col = n0 + wn * 64 + j * 32 + l31;
+      for (int j = 0; j < NJ; ++j) {
+        const int col = n0 + wn * (BN / WN) + j * 32 + l31;
         if (col < p.N)
           ((bf16 *)p.c)[o.at + col] =
               f2bf(gg::finish<bf16>(p, acc[i][j][r], o.scale));
@@ -198,7 +202,7 @@ __global__ void __launch_bounds__(256, 2) gg_tile_kernel(GroupedGemm p) {
 // ---------------------------------------------------------------------------
 template <bool SPLIT>
 __global__ void __launch_bounds__(256) gg_strip_kernel(GroupedGemm p) {
-  const gg::Tile tile = gg::tile_of(p, 16);
+  const gg::Tile tile = gg::tile_of(p, 16, blockIdx.y);
   if (tile.rows <= 0) return;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int l15 = lane & 15, g = lane >> 4;
@@ -277,7 +281,7 @@ __global__ void __launch_bounds__(256) gg_plain_kernel(GroupedGemm p) {
   constexpr int BK = 32;
   __shared__ float a_s[16][BK + 1];
   __shared__ float b_s[64][BK + 1];
-  const gg::Tile tile = gg::tile_of(p, 16);
+  const gg::Tile tile = gg::tile_of(p, 16, blockIdx.y);
   if (tile.rows <= 0) return;
   const int n0 = blockIdx.x * 64, tid = threadIdx.x;
   const int col = tid & 63, r0 = tid >> 6;

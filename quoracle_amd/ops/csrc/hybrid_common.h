@@ -107,4 +107,26 @@ template <typename T> __device__ __forceinline__ float gelu(float z) {
   }
 }
 
+// Copy 16 bytes per lane from memory straight into LDS: lane i's go to
+// `to` + 16 i, lanes that are switched off leave their place as it is.  The
+// copy is under way until the wave's vector-memory counter says otherwise, see
+// dma_barrier().  (The wait state is what a write of M0 needs before its use.)
+__device__ __forceinline__ void dma16(const void *from, void *to) {
+  const unsigned at = __builtin_amdgcn_readfirstlane(
+      (unsigned)(size_t)(__attribute__((address_space(3))) void *)to);
+  asm volatile("s_mov_b32 m0, %0\n\ts_nop 0\n\t"
+               "global_load_lds_dwordx4 %1, off"
+               :
+               : "s"(at), "v"(from)
+               : "memory", "m0");
+}
+// Barrier behind which every wave's copies so far are in LDS.
+__device__ __forceinline__ void dma_barrier() {
+  asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)\n\ts_barrier" ::: "memory");
+}
+// Barrier for LDS only: copies stay under way.
+__device__ __forceinline__ void lds_barrier() {
+  asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
+}
+
 }  // namespace hyb

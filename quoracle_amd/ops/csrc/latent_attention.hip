@@ -56,15 +56,19 @@ __device__ __forceinline__ float part_max(const float *part_m, long base,
 // Latent space.  Query rows are the flattened (token, head) pairs of a tile of
 // tokens of one sequence; a workgroup takes 16*MT of them, all of which read
 // the same cached rows.  Wave w forms the scores of 16 query rows x 16 keys
-// (mt = w % MT, kb = w / MT), and after the softmax the output columns
-// 16*(w + n*NW) of all query rows.
+// (mt = w % MT, kb = w / MT); then every wave takes the softmax of all query
+// rows for itself, in the layout of the value product's operand, and forms the
+// output columns 16*(w + n*NW).
 //   q_lat [rows, H, rank], q [rows, H, QP] with the rotated part at q_rot
 //   tile_* null: decoding, tile i is row i of sequence i at ctx[i] - 1
 //   NS > 1: partials part_m/part_l [rows, H, NS], part_acc [.., rank]
+//   pages of 2^bs_log tokens
 // Grid: (tiles, ceil(max tokens * H / (16*MT)), NS); block 64*NW.
 // ---------------------------------------------------------------------------
+template <int MT> constexpr int latent_waves() { return 2 * MT; }
+
 template <int RP, int MT>
-__global__ void __launch_bounds__(MT == 4 ? 512 : 256, MT == 1 ? 1 : 2)
+__global__ void __launch_bounds__(64 * latent_waves<MT>(), 2)
 latent_tile_kernel(bf16 *__restrict__ out, float *__restrict__ part_m,
                    float *__restrict__ part_l, float *__restrict__ part_acc,
                    const bf16 *__restrict__ q_lat, const bf16 *__restrict__ q,
@@ -75,24 +79,22 @@ latent_tile_kernel(bf16 *__restrict__ out, float *__restrict__ part_m,
                    const int *__restrict__ tile_seq,
                    const int *__restrict__ tile_pos0,
                    const float *__restrict__ sink, float scale, int H,
-                   int rank, int rot, int QP, int q_rot, int BS, int MAXB,
-                   int NS) {
-  constexpr int NW = MT == 4 ? 8 : 4;          // waves
+                   int rank, int rot, int QP, int q_rot, int bs_log,
+                   int MAXB, int NS) {
+  constexpr int NW = latent_waves<MT>();
   constexpr int NT = 64 * NW;
-  constexpr int KC = 16 * NW / MT;             // keys per step: 64, 32, 32
+  constexpr int KC = 16 * NW / MT;             // keys per step: at most 64
   constexpr int RT = 64;                       // room for the rotated part
-  constexpr int KS = RP + RT + 8;              // LDS row of a key
-  constexpr int SS = KC + 4, PS = KC + 8;
-  constexpr int NQ = RP / 32, NQR = RT / 32;
+  constexpr int SS = KC + 4;
+  constexpr int NQ = RP / 32, NQR = RT / 32, KK = KC / 32;
   constexpr int NB = (RP / 16 + NW - 1) / NW;  // output blocks per wave
-  constexpr int NV = (RP + RT) / 8;            // vectors of a key
-  constexpr int IT = (KC * NV + NT - 1) / NT;
-  __shared__ __align__(16) bf16 k_s[KC * KS];
+  // Keys in LDS: blocks of 64 columns, [KC keys][8 vectors] each; vector v of
+  // key r lies at v ^ swizzle(r), so that neither the rows of a column nor the
+  // columns of a row meet in a bank.  A copy moves 8 keys of a block.
+  constexpr int CB = (RP + RT) / 64, BLOCK = KC * 64;
+  constexpr int KG = KC / 8, IT = (CB + NW / KG - 1) / (NW / KG);
+  __shared__ __align__(16) bf16 k_s[2][CB * BLOCK];
   __shared__ __align__(16) float s_s[MT * 16 * SS];
-  __shared__ __align__(16) bf16 p_hi[MT * 16 * PS];
-  __shared__ __align__(16) bf16 p_lo[MT * 16 * PS];
-  __shared__ float m_s[MT * 16], l_s[MT * 16], alpha_s[MT * 16];
-  __shared__ int last_s[MT * 16];              // last key a row sees, or -1
 
   const int tile = blockIdx.x;
   const int q0 = tile_q0 ? tile_q0[tile] : tile;
@@ -110,36 +112,49 @@ latent_tile_kernel(bf16 *__restrict__ out, float *__restrict__ part_m,
   const int t0 = min(kv, (int)blockIdx.z * per);
   const int t1 = min(kv, t0 + per);
 
-  for (int r = tid; r < MT * 16; r += NT) {
-    const int f = f0 + r;
-    const bool live = f < qn * H;
-    last_s[r] = live ? pos0 + f / H : -1;
-    const bool start = live && sink && blockIdx.z == 0;
-    m_s[r] = start ? sink[f % H] : -INFINITY;
-    l_s[r] = start ? 1.f : 0.f;
+  int last[4];                                 // last key of a score row
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    const int f = f0 + mt * 16 + g * 4 + r;
+    last[r] = f < qn * H ? min(pos0 + f / H, t1 - 1) : -1;
   }
-  // columns behind the latent and behind the rotated part stay zero
-  for (int i = tid; i < KC * NV; i += NT) {
-    const int d = i % NV * 8;
-    if (d < RP ? d >= rank : d - RP >= rot)
-      *reinterpret_cast<uint4 *>(k_s + i / NV * KS + d) =
-          make_uint4(0, 0, 0, 0);
+  float m[MT], l[MT];                          // of row a*16 + l15
+#pragma unroll
+  for (int a = 0; a < MT; ++a) {
+    const int f = f0 + a * 16 + l15;
+    const bool start = f < qn * H && sink && blockIdx.z == 0;
+    m[a] = start ? sink[f % H] : -INFINITY;
+    l[a] = start ? 1.f : 0.f;
+  }
+  // columns behind the latent and behind the rotated part stay zero, keys
+  // behind the end finite
+  if (rank < RP || rot < RT || t1 - t0 < 2 * KC) {
+    for (int i = tid; i < CB * BLOCK / 4; i += NT)
+      reinterpret_cast<uint4 *>(k_s)[i] = make_uint4(0, 0, 0, 0);
+    __syncthreads();
   }
 
-  // Q fragments: row l15 of this wave's 16, k = g*8 + i
+  // Q fragments: row l15 of this wave's 16, k = g*8 + i; rows that are not
+  // there repeat the last one
   la_b16x8 qf[NQ + NQR];
   {
-    const int f = f0 + mt * 16 + l15;
-    const bool live = f < qn * H;
-    const long row = live ? (long)(q0 + f / H) * H + f % H : 0;
+    const int f = min(f0 + mt * 16 + l15, qn * H - 1);
+    const long row = (long)(q0 + f / H) * H + f % H;
+    const bf16 *lp = q_lat + row * rank + g * 8;
+    const bf16 *rp = q + row * QP + q_rot + g * 8;
 #pragma unroll
-    for (int kk = 0; kk < NQ + NQR; ++kk) {
+    for (int kk = 0; kk < NQ; ++kk) {
       la_b16x8 v = {};
-      const int d = kk < NQ ? kk * 32 + g * 8 : (kk - NQ) * 32 + g * 8;
-      if (live && d < (kk < NQ ? rank : rot))
-        v = *reinterpret_cast<const la_b16x8 *>(
-            kk < NQ ? q_lat + row * rank + d : q + row * QP + q_rot + d);
+      if ((RP > 64 && kk < NQ / 2) || kk * 32 + g * 8 < rank)
+        v = *reinterpret_cast<const la_b16x8 *>(lp + kk * 32);
       qf[kk] = v;
+    }
+#pragma unroll
+    for (int kk = 0; kk < NQR; ++kk) {
+      la_b16x8 v = {};
+      if (kk * 32 + g * 8 < rot)
+        v = *reinterpret_cast<const la_b16x8 *>(rp + kk * 32);
+      qf[NQ + kk] = v;
     }
   }
 
@@ -149,137 +164,149 @@ latent_tile_kernel(bf16 *__restrict__ out, float *__restrict__ part_m,
 #pragma unroll
     for (int n = 0; n < NB; ++n) o[a][n] = (la_f32x4){0.f, 0.f, 0.f, 0.f};
 
+  // This lane copies vector `unit` of key `key` of a step.  Pool rows are
+  // looked up a step ahead of the copies; -1 behind the end.
   const int width = rank + rot;
-  uint4 kr[IT];
-  auto load = [&](int start) {
+  const int key = wave % KG * 8 + (lane >> 3);
+  const int unit = (lane & 7) ^ (key >> 1 & 7);
+  const int *table = bt + (long)seq * MAXB;
+  auto find = [&](int start) {
+    const int token = start + key;
+    return token < t1 ? (table[token >> bs_log] << bs_log) +
+                            (token & ((1 << bs_log) - 1))
+                      : -1;
+  };
+  auto fetch = [&](int at, bf16 *to) {
+    if (at < 0) return;
+    const bf16 *from = pool + (long)at * width + unit * 8;
 #pragma unroll
     for (int it = 0; it < IT; ++it) {
-      const int i = tid + it * NT, key = i / NV, d = i % NV * 8;
-      uint4 v = make_uint4(0, 0, 0, 0);
-      const int token = start + key;
-      if (key < KC && token < t1 && (d < RP ? d < rank : d - RP < rot)) {
-        const long slot =
-            (long)bt[(long)seq * MAXB + token / BS] * BS + token % BS;
-        v = *reinterpret_cast<const uint4 *>(
-            pool + slot * width + (d < RP ? d : d - RP + rank));
-      }
-      kr[it] = v;
+      const int cb = wave / KG + it * (NW / KG), d = cb * 64 + unit * 8;
+      if (CB % (NW / KG) && cb >= CB) continue;
+      // more than half of the columns are always there (RP > 64)
+      const bool sure = RP > 64 && (it + 1) * (NW / KG) * 64 <= RP / 2;
+      if (sure || (d < RP ? d < rank : d - RP < rot))
+        hyb::dma16(from + (cb * 64 < RP ? cb * 64 : rank),
+                  to + cb * BLOCK + wave % KG * 512);
     }
   };
-  auto stage = [&]() {
-#pragma unroll
-    for (int it = 0; it < IT; ++it) {
-      const int i = tid + it * NT, key = i / NV, d = i % NV * 8;
-      if (key < KC && (d < RP ? d < rank : d - RP < rot))
-        *reinterpret_cast<uint4 *>(k_s + key * KS + d) = kr[it];
-    }
-  };
+  // where this lane reads: the score operand (key kb*16 + l15, even and odd
+  // 32-column steps) and the value operand (keys g*8 + l15/4 and 4 behind)
+  const int sw = l15 >> 1;
+  const int s_at[2] = {(kb * 16 + l15) * 64 + (g ^ sw) * 8,
+                       (kb * 16 + l15) * 64 + ((4 + g) ^ sw) * 8};
+  const int v_key = g * 8 + (l15 >> 2), v_unit = wave % 4 * 2 + (l15 >> 1 & 1);
+  const int v_at[2] = {
+      wave / 4 * BLOCK + v_key * 64 + (v_unit ^ (v_key >> 1 & 7)) * 8 +
+          (l15 & 1) * 4,
+      wave / 4 * BLOCK + (v_key + 4) * 64 +
+          (v_unit ^ ((v_key + 4) >> 1 & 7)) * 8 + (l15 & 1) * 4};
 
-  load(t0);
-  for (int start = t0; start < t1; start += KC) {
-    stage();
-    __syncthreads();
-    if (start + KC < t1) load(start + KC);
+  fetch(find(t0), k_s[0]);
+  int at = find(t0 + KC);
+  for (int start = t0, buf = 0; start < t1; start += KC, buf ^= 1) {
+    hyb::dma_barrier();
+    if (start + KC < t1) {
+      fetch(at, k_s[buf ^ 1]);
+      at = find(start + 2 * KC);
+    }
     {
       la_f32x4 acc = {0.f, 0.f, 0.f, 0.f};
-      const bf16 *kp = k_s + (kb * 16 + l15) * KS + g * 8;
+      const bf16 *kp = k_s[buf];
 #pragma unroll
-      for (int kk = 0; kk < NQ; ++kk)
-        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-            qf[kk], *reinterpret_cast<const la_b16x8 *>(kp + kk * 32), acc, 0,
-            0, 0);
-#pragma unroll
-      for (int kk = 0; kk < NQR; ++kk)
-        if (kk * 32 < rot)
+      for (int kk = 0; kk < NQ + NQR; ++kk)
+        if (kk <= NQ || (kk - NQ) * 32 < rot)
           acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-              qf[NQ + kk],
-              *reinterpret_cast<const la_b16x8 *>(kp + RP + kk * 32), acc, 0,
-              0, 0);
+              qf[kk],
+              *reinterpret_cast<const la_b16x8 *>(kp + kk / 2 * BLOCK +
+                                                  s_at[kk & 1]),
+              acc, 0, 0, 0);
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int row = mt * 16 + g * 4 + r, key = kb * 16 + l15;
-        s_s[row * SS + key] =
-            start + key <= last_s[row] && start + key < t1 ? acc[r] * scale
-                                                           : -INFINITY;
+      for (int r = 0; r < 4; ++r)
+        s_s[(mt * 16 + g * 4 + r) * SS + kb * 16 + l15] =
+            start + kb * 16 + l15 <= last[r] ? acc[r] * scale : -INFINITY;
+    }
+    hyb::lds_barrier();
+    la_b16x8 hi[MT][KK], lo[MT][KK];
+#pragma unroll
+    for (int a = 0; a < MT; ++a) {
+      float p[KK][8], top = -INFINITY, sum = 0.f;
+#pragma unroll
+      for (int kk = 0; kk < KK; ++kk) {
+        hyb::load_v<8>(s_s + (a * 16 + l15) * SS + kk * 32 + g * 8, p[kk]);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) top = fmaxf(top, p[kk][j]);
+      }
+      top = fmaxf(top, __shfl_xor(top, 16, 64));
+      top = fmaxf(top, __shfl_xor(top, 32, 64));
+      const float mn = fmaxf(m[a], top);
+      const float alpha = m[a] == -INFINITY ? 0.f : __expf(m[a] - mn);
+      const float base = mn == -INFINITY ? 0.f : mn;
+#pragma unroll
+      for (int kk = 0; kk < KK; ++kk) {
+        uint4 h4, l4;
+        unsigned int *hp = &h4.x, *lp = &l4.x;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          const float u = __expf(p[kk][2 * j] - base);
+          const float v = __expf(p[kk][2 * j + 1] - base);
+          sum += u + v;
+          hp[j] = pack_bf16x2(u, v);
+          float uh, vh;
+          unpack_bf16x2(hp[j], uh, vh);
+          lp[j] = pack_bf16x2(u - uh, v - vh);
+        }
+        hi[a][kk] = __builtin_bit_cast(la_b16x8, h4);
+        lo[a][kk] = __builtin_bit_cast(la_b16x8, l4);
+      }
+      sum += __shfl_xor(sum, 16, 64);
+      sum += __shfl_xor(sum, 32, 64);
+      l[a] = l[a] * alpha + sum;
+      m[a] = mn;
+      if (__any(alpha != 1.f)) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const float w = __shfl(alpha, g * 4 + r, 64);
+#pragma unroll
+          for (int n = 0; n < NB; ++n) o[a][n][r] *= w;
+        }
       }
     }
-    __syncthreads();
-    {                                          // KC/4 threads per row
-      const int row = tid / (KC / 4), c = tid % (KC / 4) * 4;
-      const float4 s = *reinterpret_cast<const float4 *>(s_s + row * SS + c);
-      float top = fmaxf(fmaxf(s.x, s.y), fmaxf(s.z, s.w));
 #pragma unroll
-      for (int w = KC / 8; w >= 1; w >>= 1)
-        top = fmaxf(top, __shfl_xor(top, w, 64));
-      const float m0 = m_s[row], mn = fmaxf(m0, top);
-      const float alpha = m0 == -INFINITY ? 0.f : __expf(m0 - mn);
-      float p[4] = {s.x, s.y, s.z, s.w}, rest[4], sum = 0.f;
-#pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        p[j] = p[j] == -INFINITY ? 0.f : __expf(p[j] - mn);
-        sum += p[j];
-        rest[j] = p[j] - bf2f(f2bf(p[j]));
-      }
-      hyb::store_v<4>(p_hi + row * PS + c, p);
-      hyb::store_v<4>(p_lo + row * PS + c, rest);
-#pragma unroll
-      for (int w = KC / 8; w >= 1; w >>= 1) sum += __shfl_xor(sum, w, 64);
-      if (c == 0) {
-        l_s[row] = l_s[row] * alpha + sum;
-        m_s[row] = mn;
-        alpha_s[row] = alpha;
-      }
-    }
-    __syncthreads();
-#pragma unroll
-    for (int a = 0; a < MT; ++a)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const float alpha = alpha_s[a * 16 + g * 4 + r];
-#pragma unroll
-        for (int n = 0; n < NB; ++n) o[a][n][r] *= alpha;
-      }
-#pragma unroll
-    for (int kk = 0; kk < KC / 32; ++kk) {
-      la_b16x8 hi[MT], lo[MT];
-#pragma unroll
-      for (int a = 0; a < MT; ++a) {
-        const int at = (a * 16 + l15) * PS + kk * 32 + g * 8;
-        hi[a] = *reinterpret_cast<const la_b16x8 *>(p_hi + at);
-        lo[a] = *reinterpret_cast<const la_b16x8 *>(p_lo + at);
-      }
+    for (int kk = 0; kk < KK; ++kk) {
 #pragma unroll
       for (int n = 0; n < NB; ++n) {
         const int col = (wave + n * NW) * 16;
         if (RP / 16 % NW && col >= RP) continue;
         // B fragment: column l15, keys g*8 + i
-        const bf16 *vp = k_s + (kk * 32 + g * 8 + (l15 >> 2)) * KS + col +
-                         (l15 & 3) * 4;
-        const la_b16x8 v = la::join4(la::read_tr(vp), la::read_tr(vp + 4 * KS));
+        const bf16 *vp = k_s[buf] + kk * 32 * 64 + n * (NW / 4) * BLOCK;
+        const la_b16x8 v = la::join4(la::read_tr(vp + v_at[0]),
+                                     la::read_tr(vp + v_at[1]));
 #pragma unroll
         for (int a = 0; a < MT; ++a) {
-          o[a][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(hi[a], v, o[a][n],
-                                                            0, 0, 0);
-          o[a][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(lo[a], v, o[a][n],
-                                                            0, 0, 0);
+          o[a][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(hi[a][kk], v,
+                                                            o[a][n], 0, 0, 0);
+          o[a][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(lo[a][kk], v,
+                                                            o[a][n], 0, 0, 0);
         }
       }
     }
-    __syncthreads();
   }
-  if (t0 >= t1) __syncthreads();               // m_s and l_s are written
 #pragma unroll
-  for (int a = 0; a < MT; ++a)
+  for (int a = 0; a < MT; ++a) {
+    const float inv_a = l[a] > 0.f ? 1.f / l[a] : 0.f;
+    const int fl = f0 + a * 16 + l15;
+    if (NS > 1 && wave == 0 && g == 0 && fl < qn * H) {
+      const long row = (long)(q0 + fl / H) * H + fl % H;
+      part_m[row * NS + blockIdx.z] = m[a];
+      part_l[row * NS + blockIdx.z] = l[a];
+    }
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      const int lr = a * 16 + g * 4 + r, f = f0 + lr;
+      const float inv = __shfl(inv_a, g * 4 + r, 64);
+      const int f = f0 + a * 16 + g * 4 + r;
       if (f >= qn * H) continue;
       const long row = (long)(q0 + f / H) * H + f % H;
-      if (NS > 1 && wave == 0 && l15 == 0) {
-        part_m[row * NS + blockIdx.z] = m_s[lr];
-        part_l[row * NS + blockIdx.z] = l_s[lr];
-      }
-      const float l = l_s[lr], inv = l > 0.f ? 1.f / l : 0.f;
 #pragma unroll
       for (int n = 0; n < NB; ++n) {
         const int col = (wave + n * NW) * 16 + l15;
@@ -290,9 +317,12 @@ latent_tile_kernel(bf16 *__restrict__ out, float *__restrict__ part_m,
           out[row * rank + col] = f2bf(o[a][n][r] * inv);
       }
     }
+  }
 }
 
-// Grid: (rows, H); block 128.  LDS NS floats, dynamic.
+// Join the NS partial softmaxes of a row: a workgroup takes 128 columns, each
+// of its four groups of 32 lanes every fourth part.
+// Grid: (rows, H, ceil(rank / 128)); block 128; dynamic LDS NS floats.
 __global__ void __launch_bounds__(128)
 latent_combine_kernel(bf16 *__restrict__ out, const float *__restrict__ part_m,
                       const float *__restrict__ part_l,
@@ -300,6 +330,7 @@ latent_combine_kernel(bf16 *__restrict__ out, const float *__restrict__ part_m,
                       int NS) {
   extern __shared__ float w_s[];
   __shared__ float scratch[2];
+  __shared__ __align__(16) float sum_s[4][128];
   const long row = (long)blockIdx.x * H + blockIdx.y, base = row * NS;
   const float m = la::part_max(part_m, base, 1, NS, scratch);
   float l = 0.f;
@@ -311,18 +342,24 @@ latent_combine_kernel(bf16 *__restrict__ out, const float *__restrict__ part_m,
   }
   l = block_sum(l, scratch);                   // its barriers publish w_s
   const float inv = l > 0.f ? 1.f / l : 0.f;
-  for (int d = threadIdx.x * 4; d < rank; d += 512) {
-    float o[4] = {0.f, 0.f, 0.f, 0.f}, v[4];
-    for (int i = 0; i < NS; ++i) {
-      if (w_s[i] == 0.f) continue;
+  const int grp = threadIdx.x >> 5, c = (threadIdx.x & 31) * 4;
+  const int d = blockIdx.z * 128 + c;
+  float o[4] = {0.f, 0.f, 0.f, 0.f}, v[4];
+  if (d < rank) {
+#pragma unroll 4
+    for (int i = grp; i < NS; i += 4) {
       hyb::load_v<4>(part_acc + (base + i) * rank + d, v);
 #pragma unroll
       for (int j = 0; j < 4; ++j) o[j] = fmaf(w_s[i], v[j], o[j]);
     }
-#pragma unroll
-    for (int j = 0; j < 4; ++j) o[j] *= inv;
-    hyb::store_v<4>(out + row * rank + d, o);
   }
+  hyb::store_v<4>(&sum_s[grp][c], o);
+  __syncthreads();
+  if (grp || d >= rank) return;
+#pragma unroll
+  for (int j = 0; j < 4; ++j)
+    o[j] = (o[j] + sum_s[1][c + j] + sum_s[2][c + j] + sum_s[3][c + j]) * inv;
+  hyb::store_v<4>(out + row * rank + d, o);
 }
 
 // ---------------------------------------------------------------------------

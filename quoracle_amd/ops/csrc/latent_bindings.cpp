@@ -142,24 +142,31 @@ bool gg_vectors_ok(const GroupedGemm &p) {
 
 // Rows per tile that suit `rows` rows per group on average.
 int gg_tile_rows(bool vec, long rows) {
-  return !vec || rows <= 32 ? 16 : rows <= 96 ? 64 : 128;
+  return !vec || rows <= 32 ? 16 : rows <= 96 ? 64 : rows < 1024 ? 128 : 256;
 }
 
 // `tiles` row tiles of BM rows (of every group, if there is no tile list).
 template <typename A>
-void gg_launch(const GroupedGemm &p, int BM, long tiles, long groups,
-               bool vec) {
+void gg_launch(GroupedGemm p, int BM, long tiles, long groups, bool vec) {
   if (tiles == 0 || groups == 0 || p.N == 0) return;
   TORCH_CHECK(tiles <= 65535 && groups <= 65535, "grouped product grid");
+  p.row_tiles = tiles;
   auto run = [&](auto kernel, int cols) {
     kernel<<<dim3((p.N + cols - 1) / cols, tiles, groups), dim3(256), 0,
              current_stream()>>>(p);
     HIP_CHECK_KERNEL();
   };
+  auto run_tiles = [&](auto kernel, int cols, int threads) {
+    const long all = (p.N + cols - 1) / cols * tiles;
+    TORCH_CHECK(all < 1L << 31, "grouped product grid");
+    kernel<<<dim3(all, 1, groups), dim3(threads), 0, current_stream()>>>(p);
+    HIP_CHECK_KERNEL();
+  };
   if constexpr (sizeof(A) == 2) {
     if (vec) {
-      if (BM == 128) run(gg_tile_kernel<128>, 128);
-      else if (BM == 64) run(gg_tile_kernel<64>, 128);
+      if (BM == 256) run_tiles(gg_tile_kernel<256, 256, 2, 4>, 256, 512);
+      else if (BM == 128) run_tiles(gg_tile_kernel<128, 128, 2, 2>, 128, 256);
+      else if (BM == 64) run_tiles(gg_tile_kernel<64, 128, 2, 2>, 128, 256);
       else if (p.K > 256) run(gg_strip_kernel<true>, 32);
       else run(gg_strip_kernel<false>, 128);
       return;
@@ -193,7 +200,8 @@ void head_product(const Tensor &c, const Tensor &a, int64_t a_off,
     p.N = N;
     p.K = K;
     const bool vec = gg_vectors_ok(p) && a_off % 8 == 0;
-    const int BM = gg_tile_rows(vec && sizeof(A) == 2, rows);
+    // few columns: short tiles, so that there are enough of them
+    const int BM = rows <= 64 ? 16 : gg_tile_rows(vec && sizeof(A) == 2, rows);
     gg_launch<A>(p, BM, (rows + BM - 1) / BM, H, vec);
   });
 }
@@ -204,7 +212,7 @@ struct LatentDims {
   int H, QP, dim, rot, rank, vdim, BS, MAXB;
 };
 
-// Workgroups that fill the chip twice over.
+// Workgroups that fill the chip, two on a CU.
 constexpr long LATENT_GROUPS = 512;
 
 // Rows of one launch in the latent space: decode rows (tiles undefined), or
@@ -215,10 +223,11 @@ void latent_tiles(const Tensor &o, const Tensor &q_lat, const Tensor &q,
                   const Tensor *tiles, long n_tiles, int tokens, long seen) {
   if (n_tiles == 0) return;
   const long rows = (long)tokens * d.H;        // flattened rows of a tile
-  const int MT = rows <= 16 ? 1 : rows <= 32 ? 2 : 4;
+  const int MT = rows <= 32 ? 2 : 4;
   const long parts = (rows + 16 * MT - 1) / (16 * MT);
   const long ns = std::max<long>(
-      1, std::min<long>({LATENT_GROUPS / (n_tiles * parts), seen / 128, 64}));
+      1, std::min<long>({LATENT_GROUPS * 2 / MT / (n_tiles * parts), seen / 64,
+                         64}));
   Tensor pm, pl, pa;
   if (ns > 1) {
     auto opts = q.options().dtype(torch::kFloat32);
@@ -229,7 +238,7 @@ void latent_tiles(const Tensor &o, const Tensor &q_lat, const Tensor &q,
   auto run = [&](auto rp, auto mt) {
     constexpr int RP = decltype(rp)::value, M = decltype(mt)::value;
     latent_tile_kernel<RP, M>
-        <<<dim3(n_tiles, parts, ns), dim3(M == 4 ? 512 : 256), 0,
+        <<<dim3(n_tiles, parts, ns), dim3(64 * latent_waves<M>()), 0,
            current_stream()>>>(
             ptr<bf16>(o), ns > 1 ? fptr(pm) : nullptr,
             ns > 1 ? fptr(pl) : nullptr, ns > 1 ? fptr(pa) : nullptr,
@@ -237,12 +246,11 @@ void latent_tiles(const Tensor &o, const Tensor &q_lat, const Tensor &q,
             tiles ? nullptr : iptr(ctx), tiles ? iptr(tiles[0]) : nullptr,
             tiles ? iptr(tiles[1]) : nullptr, tiles ? iptr(tiles[2]) : nullptr,
             tiles ? iptr(tiles[3]) : nullptr, sink ? fptr(*sink) : nullptr,
-            (float)scale, d.H, d.rank, d.rot, d.QP, d.dim, d.BS, d.MAXB,
-            (int)ns);
+            (float)scale, d.H, d.rank, d.rot, d.QP, d.dim,
+            __builtin_ctz(d.BS), d.MAXB, (int)ns);
   };
   auto sized = [&](auto rp) {
-    if (MT == 1) run(rp, Int<1>());
-    else if (MT == 2) run(rp, Int<2>());
+    if (MT == 2) run(rp, Int<2>());
     else run(rp, Int<4>());
   };
   if (d.rank <= 64) sized(Int<64>());
@@ -255,8 +263,8 @@ void latent_tiles(const Tensor &o, const Tensor &q_lat, const Tensor &q,
   const long first = tiles ? ctx.size(0) : 0;
   const long n = tiles ? o.size(0) - first : ctx.size(0);
   const long at = first * d.H;
-  latent_combine_kernel<<<dim3(n, d.H), dim3(128), ns * sizeof(float),
-                          current_stream()>>>(
+  latent_combine_kernel<<<dim3(n, d.H, (d.rank + 127) / 128), dim3(128),
+                          ns * sizeof(float), current_stream()>>>(
       ptr<bf16>(o) + at * d.rank, fptr(pm) + at * ns, fptr(pl) + at * ns,
       fptr(pa) + at * ns * d.rank, d.H, d.rank, (int)ns);
   HIP_CHECK_KERNEL();
@@ -348,7 +356,7 @@ void latent_attend(const Tensor &out, const Tensor &q, const Tensor &pool,
   // a batch with portions that names neither short tiles nor contexts is one
   // of a model with other layers that the matrix kernels do not take
   const bool tiles = q.scalar_type() == torch::kBFloat16 && d.rank <= 512 &&
-                     d.rot <= 64 &&
+                     d.rot <= 64 && (d.BS & (d.BS - 1)) == 0 &&
                      (T == b.n_decode || b.n_latent > b.n_decode ||
                       b.has("ctx_slots"));
   const long n = tiles ? b.n_latent : T;
@@ -452,12 +460,12 @@ void moe_experts(Tensor y, Tensor h, Tensor ids, Tensor weights, Tensor up,
     const bool vec = sizeof(A) == 2 && n % 8 == 0 && ff % 8 == 0;
     const int BM = gg_tile_rows(vec, (S + E - 1) / E);
     const long nt = S / BM + std::min<long>(E, S);
-    auto list = torch::empty({S + 3 * nt}, ids.options());
+    auto list = torch::empty({S + 3 * nt + 1}, ids.options());
     int *rows = list.data_ptr<int>();
-    int *tg = rows + S, *tr0 = tg + nt, *trn = tr0 + nt;
+    int *tg = rows + S, *tr0 = tg + nt, *trn = tr0 + nt, *count = trn + nt;
     moe_order_kernel<<<dim3(1), dim3(1024), 3 * E * sizeof(int),
-                       current_stream()>>>(rows, tg, tr0, trn, iptr(ids),
-                                           (int)S, E, BM, (int)nt);
+                       current_stream()>>>(rows, tg, tr0, trn, count,
+                                           iptr(ids), (int)S, E, BM, (int)nt);
     HIP_CHECK_KERNEL();
     auto act = torch::empty({S, ff}, h.options());
     GroupedGemm p{};
@@ -471,6 +479,7 @@ void moe_experts(Tensor y, Tensor h, Tensor ids, Tensor weights, Tensor up,
     p.tile_group = tg;
     p.tile_row0 = tr0;
     p.tile_rows = trn;
+    p.tile_count = count;
     p.rows = rows;
     p.a_div = top;
     p.scale = fptr(weights);

@@ -91,20 +91,29 @@ moe_route_mfma_kernel(int *__restrict__ ids, float *__restrict__ weights,
       b_ok[j] = c0 + 16 * j + l15 < cols;
       bp[j] = router + (b_ok[j] ? (long)(c0 + 16 * j + l15) * n : 0) + g * 8;
     }
-    for (int k = wave * 32; k < n; k += 256) {
-      const bool in = k + g * 8 < n;
-      uint4 av = make_uint4(0, 0, 0, 0), bv[4];
-      if (in && a_ok) av = *reinterpret_cast<const uint4 *>(ap + k);
+    constexpr int U = 4;                     // steps under way
+    for (int k0 = wave * 32; k0 < n; k0 += 256 * U) {
+      uint4 av[U], bv[U][4];
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
-        bv[j] = in && b_ok[j] ? *reinterpret_cast<const uint4 *>(bp[j] + k)
-                              : make_uint4(0, 0, 0, 0);
+      for (int u = 0; u < U; ++u) {
+        const int k = k0 + u * 256;
+        const bool in = k + g * 8 < n;
+        av[u] = in && a_ok ? *reinterpret_cast<const uint4 *>(ap + k)
+                           : make_uint4(0, 0, 0, 0);
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
-        if (c0 + 16 * j < cols)
-          acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-              __builtin_bit_cast(gg_b16x8, av),
-              __builtin_bit_cast(gg_b16x8, bv[j]), acc[j], 0, 0, 0);
+        for (int j = 0; j < 4; ++j)
+          bv[u][j] = in && b_ok[j]
+                         ? *reinterpret_cast<const uint4 *>(bp[j] + k)
+                         : make_uint4(0, 0, 0, 0);
+      }
+#pragma unroll
+      for (int u = 0; u < U; ++u)
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          if (c0 + 16 * j < cols)
+            acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+                __builtin_bit_cast(gg_b16x8, av[u]),
+                __builtin_bit_cast(gg_b16x8, bv[u][j]), acc[j], 0, 0, 0);
     }
 #pragma unroll
     for (int j = 0; j < 4; ++j)
@@ -132,12 +141,13 @@ moe_route_mfma_kernel(int *__restrict__ ids, float *__restrict__ weights,
 
 // ---------------------------------------------------------------------------
 // Slots (token * top + k) in the order of their experts, and the list of row
-// tiles (BM rows of one expert each); unused tiles get 0 rows.
+// tiles (BM rows of one expert each) and its length; unused tiles get 0 rows.
 // Grid: (1); block 1024; dynamic LDS 3 * E ints.
 // ---------------------------------------------------------------------------
 __global__ void __launch_bounds__(1024)
 moe_order_kernel(int *__restrict__ rows, int *__restrict__ tile_group,
                  int *__restrict__ tile_row0, int *__restrict__ tile_rows,
+                 int *__restrict__ tile_count,
                  const int *__restrict__ ids, int S, int E, int BM,
                  int n_tiles) {
   extern __shared__ int order_s[];
@@ -165,7 +175,7 @@ moe_order_kernel(int *__restrict__ rows, int *__restrict__ tile_group,
       at += __shfl(cs, 63, 64);
       tl += __shfl(ts, 63, 64);
     }
-    if (threadIdx.x == 0) used = tl;
+    if (threadIdx.x == 0) *tile_count = used = tl;
   }
   __syncthreads();
   for (int e = threadIdx.x; e < E; e += 1024)

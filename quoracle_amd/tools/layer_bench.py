@@ -126,8 +126,10 @@ def decode(sides: List[Side], device, batch: int, context: int,
             s.feed([(i, [5], ()) for i in ids])
 
             def run():
+                # a different token for each, so that experts differ too
                 for t in range(steps):
-                    s.feed([(i, [t % VOCAB], ()) for i in ids])
+                    s.feed([(i, [(131 * t + 977 * k) % VOCAB], ())
+                            for k, i in enumerate(ids)])
             best[s.name] = min(best[s.name], _timed(device, run) / steps)
     for s in sides:
         s.drop(ids)

@@ -356,7 +356,7 @@ def test_captured_decode_equals_eager(cases, name, dtype):
         got, want = (e.step_entries(
             case.path, [(r, t, range(len(t))) for r, t in part], toks)
             for e in (graph, eager))
-        assert error(got, want) < tolerance(dtype) / 5
+        assert error(got, want) < tolerance(dtype) / 3
         torch.randn(512, 512, device="cuda").sum().item()
     assert graph.stats.get("graph_steps", 0) > 20
     assert "graph_steps" not in eager.stats
